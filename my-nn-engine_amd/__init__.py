@@ -55,7 +55,11 @@ class ModelConfig(C.Structure):
                 ("ffn", _i), ("vocab", _i), ("max_seq", _i), ("eps", _f), ("rope_theta", _f), ("dtype", _i),
                 ("seq_q", _i), ("batch", _i), ("weights_int8", _i), ("quant_kv_cache", _i),
                 ("quantize_activations", _i), ("streaming_kv", _i), ("gemm_tile", _i), ("unfused_decode", _i),
-                ("handover_spin_limit", _i), ("weight_arena", _i), ("kv_page_rows", _i), ("qkv_bias", _i)]
+                ("handover_spin_limit", _i), ("weight_arena", _i), ("kv_page_rows", _i), ("qkv_bias", _i), ("arch", _i)]
+
+
+class EngineOptions(C.Structure):
+    _fields_ = [("dtype", _i), ("max_seq", _i), ("max_tokens", _i), ("prefill_rows", _i), ("page_rows", _i)]
 
 
 class KernelTime(C.Structure):
@@ -128,6 +132,23 @@ SIGNATURES = {
     "alloc_pinned": (_vp, [_sz]),
     "free_pinned": (None, [_vp]),
     "mynn_model_step": (_i, [_vp, _vp, _vp, _i64, _i64, _vp, _vp]),
+    "mynn_model_step_rows": (_i, [_vp, _vp, _i, _i64, _i, _i, _vp, _vp]),
+    "mynn_model_vocab": (_i, [_vp]),
+    "mynn_arch_open": (_i, [C.c_char_p]),
+    "mynn_arch_name": (C.c_char_p, [_i]),
+    "mynn_arch_config": (_i, [_i, _i, _i, _i, _i, C.POINTER(ModelConfig)]),
+    "mynn_arch_tensor_count": (_i, [_i]),
+    "mynn_arch_tensor": (C.c_char_p, [_i, _i, C.POINTER(_i64), C.POINTER(_i)]),
+    "mynn_arch_state_count": (_i, [_i]),
+    "mynn_arch_state_row_bytes": (_sz, [_i, _i, _i]),
+    "mynn_engine_open": (_vp, [C.c_char_p, C.POINTER(EngineOptions)]),
+    "mynn_engine_vocab": (_i, [_vp]),
+    "mynn_engine_session": (_vp, [_vp, _i64]),
+    "mynn_engine_free_rows": (_i, [_vp]),
+    "mynn_engine_close": (_i, [_vp]),
+    "mynn_llm_decode_state": (_vp, [_vp]),
+    "mynn_llm_prefill_state": (_vp, [_vp]),
+    "mynn_llm_feed": (_i, [_vp, _vp, _sz, _vp, _sz, _vp]),
     "mynn_model_step_streaming": (_i, [_vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _vp, _vp, _vp]),
     "mynn_model_handover_failures": (_i, [_vp]),
     "mynn_model_set_handover_rearm": (_i, [_vp, _i]),
@@ -899,11 +920,126 @@ class Decoder:
         return {"arena_bytes": a.value, "launches_per_step": n.value, "graph": bool(g.value)}
 
 
+class Arch:
+    """A config.json read by the model registry (mynn_arch_open)."""
+
+    def __init__(self, path):
+        self.id = lib().mynn_arch_open(str(path).encode())
+        if self.id < 0:
+            raise MynnError("mynn error %d: %s" % (self.id, lib().mynn_last_error().decode()))
+        self.name = lib().mynn_arch_name(self.id).decode()
+
+    def config(self, dtype, max_seq, seq_q=1, batch=1):
+        cfg = ModelConfig()
+        check(lib().mynn_arch_config(self.id, dtype, max_seq, seq_q, batch, C.byref(cfg)))
+        return cfg
+
+    def tensors(self):
+        """[(name, shape)] in `initializer` order"""
+        out = []
+        for i in range(lib().mynn_arch_tensor_count(self.id)):
+            shape, nd = (_i64 * 8)(), _i()
+            name = lib().mynn_arch_tensor(self.id, i, shape, C.byref(nd)).decode()
+            out.append((name, tuple(shape[d] for d in range(nd.value))))
+        return out
+
+    def state_row_bytes(self, dtype):
+        return [lib().mynn_arch_state_row_bytes(self.id, i, dtype) for i in range(lib().mynn_arch_state_count(self.id))]
+
+
+class LayeredDecoder(object):
+    """An executor of a layered architecture over a dict of cuda tensors (checkpoint names, cfg dtype).
+
+    state: the session's buffers (shared by its prefill and decode executors), made when None; kv_pages: a KvPages, state
+    then holds pool pages (`layered_state(..., n_pages=)`)."""
+
+    def __init__(self, arch, weights, dtype, max_seq, seq_q=1, batch=1, state=None, kv_pages=None, weight_set=None):
+        import torch
+
+        self.arch, self.cfg = arch, arch.config(dtype, max_seq, seq_q, batch)
+        self.cfg.kv_page_rows = kv_pages.pool.page_rows if kv_pages is not None else 0
+        self.weights, self.kv_pages = weights, kv_pages
+        self.state = state if state is not None else layered_state(arch, dtype, batch * max_seq)
+        ptrs = [t.data_ptr() for t in self.state] + ([kv_pages.handle] if kv_pages is not None else [])
+        self._state = (_vp * len(ptrs))(*ptrs)
+        self._init = (_vp * len(arch.tensors()))(*[_ptr(weights[n]) for n, _ in arch.tensors()])
+        self.weight_set = weight_set
+        torch.cuda.synchronize()
+        if weight_set is None:
+            self.handle = lib().mynn_model_create(C.byref(self.cfg), self._init, self._state)
+        else:
+            self.handle = lib().mynn_model_create_shared(C.byref(self.cfg), weight_set, self._state)
+        if not self.handle:
+            raise MynnError("model_create failed: %s" % lib().mynn_last_error().decode())
+
+    close = Decoder.close
+    __del__ = Decoder.__del__
+    stats = Decoder.stats
+    decode_loop = Decoder.decode_loop
+    profile = Decoder.profile
+    profile_step = Decoder.profile_step
+
+    def step_rows(self, ids, rows, past_len, first=None, n_logits=1):
+        """`rows` new tokens per sequence; returns (next tokens or None, f32 logits [batch, n_logits, vocab])."""
+        import numpy as np
+
+        if first is None:
+            first = rows - n_logits
+        ids = np.ascontiguousarray(np.asarray(ids, np.int64).ravel())
+        assert ids.size == self.cfg.batch * rows
+        out = np.empty((self.cfg.batch, n_logits, self.cfg.vocab), np.float32)
+        want_next = n_logits > 0 and first + n_logits == rows
+        nxt = (C.c_int32 * self.cfg.batch)()
+        check(lib().mynn_model_step_rows(self.handle, ids.ctypes.data_as(_vp), rows, int(past_len), first, n_logits,
+                                         nxt if want_next else None, out.ctypes.data_as(_vp) if n_logits else None))
+        return (list(nxt) if want_next else None), out
+
+
+def layered_state(arch, dtype, rows, fill=0):
+    """Session-state buffers of `rows` cache rows each (batch * max_seq, or n_pages * page_rows of a pool)."""
+    import torch
+
+    return [torch.full((rows * b,), fill, dtype=torch.uint8, device="cuda") for b in arch.state_row_bytes(dtype)]
+
+
+class Engine:
+    """One checkpoint on the device (mynn_engine): the model chosen by config.json, sessions over shared weights and pages."""
+
+    def __init__(self, model_dir, dtype, max_tokens, max_seq=0, prefill_rows=0, page_rows=0):
+        import torch
+
+        torch.cuda.synchronize()
+        opt = EngineOptions(dtype, max_seq, max_tokens, prefill_rows, page_rows)
+        self.handle = lib().mynn_engine_open(str(model_dir).encode(), C.byref(opt))
+        if not self.handle:
+            raise MynnError(lib().mynn_last_error().decode())
+        self.vocab = lib().mynn_engine_vocab(self.handle)
+
+    def session(self, eos=-1):
+        return LlmSession(engine=self, eos=eos)
+
+    @property
+    def free_rows(self):
+        return lib().mynn_engine_free_rows(self.handle)
+
+    def close(self):
+        if getattr(self, "handle", None) and _lib is not None:
+            check(_lib.mynn_engine_close(self.handle))
+            self.handle = None
+
+
 class LlmSession:
     """crates/llm LlmSession: decode model + optional prefill model over shared weights and KV."""
 
-    def __init__(self, decoder, prefill=None, eos=-1, streaming=None):
-        """streaming = (sink, window): DecodeKind::LlamaStreaming; the models must have been built with streaming_kv."""
+    def __init__(self, decoder=None, prefill=None, eos=-1, streaming=None, engine=None):
+        """streaming = (sink, window): DecodeKind::LlamaStreaming; the models must have been built with streaming_kv.
+        engine: a session of an Engine, which then makes the models itself."""
+        if engine is not None:
+            self.engine = engine
+            self.handle = lib().mynn_engine_session(engine.handle, int(eos))
+            if not self.handle:
+                raise MynnError(lib().mynn_last_error().decode())
+            return
         self.decoder, self.prefill = decoder, prefill
         pl = prefill.cfg.seq_q if prefill is not None else 0
         self.handle = lib().mynn_llm_create(decoder.handle, prefill.handle if prefill is not None else None, pl,
@@ -934,6 +1070,17 @@ class LlmSession:
     @past_len.setter
     def past_len(self, v):
         lib().mynn_llm_set_past_len(self.handle, int(v))
+
+    def feed(self, ids, want):
+        """Feeds given tokens; f32 logits [len(want), vocab] at the places `want` (rising) among them."""
+        import numpy as np
+
+        p = np.ascontiguousarray(np.asarray(ids, np.int64))
+        w = np.ascontiguousarray(np.asarray(want, np.int64))
+        state = lib().mynn_llm_decode_state(self.handle)
+        out = np.empty((w.size, lib().mynn_model_vocab(state)), np.float32)
+        check(lib().mynn_llm_feed(self.handle, p.ctypes.data_as(_vp), p.size, w.ctypes.data_as(_vp), w.size, out.ctypes.data_as(_vp)))
+        return out
 
     def generate_ids(self, prompt_ids, max_new_tokens):
         import numpy as np

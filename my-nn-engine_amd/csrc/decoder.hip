@@ -12,14 +12,9 @@
 // One stream, one arena allocated at init; weights and KV buffers stay caller-owned.
 #include <algorithm>
 #include <cstdio>
-#include <cstring>
-#include <map>
-#include <mutex>
-#include <vector>
 
-#include "attention.h"
-#include "kernels.h"
-#include "kv_pages.h"
+#include "executor.h"
+#include "model_spec.h"
 
 namespace mynn {
 
@@ -74,55 +69,14 @@ __global__ void heads_to_tokens_kernel(T *out, const T *in, int H, int S, int D)
     out[i] = in[((size_t)h * S + s) * D + d];
 }
 
-struct Lin {
-    const void *w = nullptr;      // int8 [N,K] when scale != nullptr, else T [N,K]
-    const void *scale = nullptr;  // T [N]
-    int N = 0, K = 0;
-};
-
-struct Layer {
-    const void *norm1 = nullptr, *norm2 = nullptr;
-    Lin qkv, o, gate, up, gu, down;  // qkv = rows of q,k,v concatenated; gu = gate/up rows interleaved
-    void *k_cache = nullptr, *v_cache = nullptr;
-    void *k_scale = nullptr, *v_scale = nullptr;  // int8 KV cache: per-token scales [B,Hkv,max_seq]
-    // (everything below points into the model's WeightSet)
-    void *qkv_b = nullptr;  // qkv_bias: the q, k, v projection biases concatenated [QD + 2 KD], T
-    // prefill executors: weights dequantised once to the 16-bit type, [N, Kp] (wt_gu: gate/up in groups of 32)
-    void *wt_qkv = nullptr, *wt_o = nullptr, *wt_gu = nullptr, *wt_down = nullptr;
-    // few-row executors: int8 weights re-tiled so that a wave streams them sequentially
-    void *pk_qkv = nullptr, *pk_o = nullptr, *pk_gu = nullptr, *pk_down = nullptr;
-    // W8A8 prefill executors: int8 gate/up rows and their scales interleaved in groups of 32 (SwiGLU store)
-    void *q8_gu = nullptr, *q8_gu_scale = nullptr;
-};
-
-// Every copy the library derives from a checkpoint's weights, made at most once and shared by the executors of a
-// session (prefill, decode, few-row): the q|k|v and gate/up repacks, the 16-bit resident copy of the matrix-core path,
-// the tiled int8 copy of the few-row path, the W8A8 gate/up interleave.  A copy is made by the first executor that
-// needs it (under the set's mutex) and lives until the last holder -- the caller's handle or a model -- lets go.
-struct WeightLayer {
-    void *qkv_w = nullptr, *qkv_s = nullptr, *gu_w = nullptr, *gu_s = nullptr, *qkv_b = nullptr;
-    void *wt_qkv = nullptr, *wt_o = nullptr, *wt_gu = nullptr, *wt_down = nullptr;
-    void *pk_qkv = nullptr, *pk_o = nullptr, *pk_gu = nullptr, *pk_down = nullptr;
-    void *q8_gu = nullptr, *q8_gu_scale = nullptr;
-};
-struct WeightSet {
-    std::mutex mu;
-    int refs = 1;
-    // what the copies depend on: the shapes, the storage type, the caller's buffers
-    int n_layers = 0, hidden = 0, n_heads = 0, n_kv_heads = 0, head_dim = 0, ffn = 0, vocab = 0, dtype = 0, int8_weights = 0, qkv_bias = 0;
-    std::vector<void *> initializer;
-    std::vector<WeightLayer> layers;
-    void *wt_lm_head = nullptr, *pk_lm_head = nullptr;
-    bool repacked = false, resident16 = false, packed8 = false, q8 = false;
-    size_t bytes_repack = 0, bytes_resident16 = 0, bytes_packed8 = 0, bytes_q8 = 0;
-};
 static size_t initializer_count(const mynn_model_config &c) {
+    if (c.arch) return arch_spec(c.arch)->tensors.size();
     return 2 + (size_t)c.n_layers * (2 + 14 + (c.qkv_bias ? 3 : 0)) + 1 + 2;
 }
 static WeightSet *weight_set_new(const mynn_model_config &c, void **init) {
     WeightSet *w = new WeightSet;
     w->n_layers = c.n_layers; w->hidden = c.hidden; w->n_heads = c.n_heads; w->n_kv_heads = c.n_kv_heads; w->head_dim = c.head_dim;
-    w->ffn = c.ffn; w->vocab = c.vocab; w->dtype = c.dtype; w->int8_weights = c.weights_int8; w->qkv_bias = c.qkv_bias;
+    w->ffn = c.ffn; w->vocab = c.vocab; w->dtype = c.dtype; w->int8_weights = c.weights_int8; w->qkv_bias = c.qkv_bias; w->arch = c.arch;
     w->initializer.assign(init, init + initializer_count(c));
     w->layers.resize(c.n_layers);
     return w;
@@ -130,7 +84,7 @@ static WeightSet *weight_set_new(const mynn_model_config &c, void **init) {
 static bool weight_set_fits(const WeightSet &w, const mynn_model_config &c) {
     return w.n_layers == c.n_layers && w.hidden == c.hidden && w.n_heads == c.n_heads && w.n_kv_heads == c.n_kv_heads &&
            w.head_dim == c.head_dim && w.ffn == c.ffn && w.vocab == c.vocab && w.dtype == c.dtype && w.int8_weights == c.weights_int8 &&
-           w.qkv_bias == c.qkv_bias;
+           w.qkv_bias == c.qkv_bias && w.arch == c.arch;
 }
 static void weight_set_release(WeightSet *w) {
     if (!w) return;
@@ -144,116 +98,13 @@ static void weight_set_release(WeightSet *w) {
             if (p) (void)hipFree(p);
     if (w->wt_lm_head) (void)hipFree(w->wt_lm_head);
     if (w->pk_lm_head) (void)hipFree(w->pk_lm_head);
+    layered_weights_free(w->layered);
     delete w;
 }
-
-struct Launch {
-    const char *name;
-    double bytes;
-    double flops;
-};
-
-struct Model {
-    mynn_model_config cfg{};
-    bool quant = true;
-    Lin embed, lm_head;
-    const void *final_norm = nullptr;
-    std::vector<Layer> layers;
-    void *wt_lm_head = nullptr, *pk_lm_head = nullptr;
-    WeightSet *wset = nullptr;  // the derived weight copies (shared with the session's other executors)
-    bool w8a8_fused = false;  // W8A8 with the large int8 tiles: norm+quantise, residual and SwiGLU ride on the launches
-    bool qgemv1 = false;      // W8A8 at batch 1: norm, quantiser, int8 GEMV and residual / SwiGLU of a linear in one launch
-    bool resident16 = false;  // the wt_* copies exist and the matrix-core path with fused stores is used
-    bool skinny = false;      // 16..64 rows: int8 weights streamed once through the few-row matrix-core kernel
-    float *skinny_scratch = nullptr;
-    void *cos_t = nullptr, *sin_t = nullptr;
-    // arena
-    char *arena = nullptr;
-    size_t arena_bytes = 0;
-    void *x = nullptr, *x2 = nullptr, *nrm = nullptr, *qkv = nullptr, *q = nullptr, *attn = nullptr, *g = nullptr,
-         *u = nullptr, *hmid = nullptr, *proj = nullptr, *logits = nullptr;
-    int8_t *a8 = nullptr;    // W8A8: the current linear's activation rows as int8 [rows, max(H, QD, F)]
-    void *a8_scale = nullptr;  // and their per-row scales [rows]
-    int64_t *d_ids = nullptr, *d_pos = nullptr;
-    int32_t *d_past = nullptr, *d_active = nullptr, *d_next = nullptr, *d_tokens = nullptr, *d_step = nullptr;
-    void *attn_scratch = nullptr;
-    int nsplit = 1, slice = 0, heads_per_wg = 1;
-    int token_cap = 0;
-    // host staging (pinned)
-    char *h_stage = nullptr;
-    size_t stage_bytes = 0, next_stage = 256;
-    hipStream_t stream = nullptr;
-    hipGraph_t graph = nullptr;
-    hipGraphExec_t graph_exec = nullptr;
-    bool use_graph = false;
-    int launches = 0;
-    // batch-1 decode: projection and attention share a launch; m.qkv is then the hand-over vector between them
-    // (all 0xFFFF between uses) and d_past[3] the error word of its bounded waits
-    // the device-resident loop replays kLoopSteps steps per graph launch where it can (a graph launch costs the device a
-    // few microseconds of its own, a tenth of a batch-1 step's launches)
-    hipGraph_t graph_loop = nullptr;
-    hipGraphExec_t graph_loop_exec = nullptr;
-    bool qkv_attn = false;
-    bool lm_argmax = false;       // ... and the lm_head launch finds the greedy token and moves the loop state on
-    uint64_t *lm_cand = nullptr;  // its candidate words (all ~0 between launches)
-    int spin_limit = 400000;      // polls a consumer role makes before it gives up and raises the error word
-    int handover_failures = 0;    // steps whose hand-over gave up; the executor then rebuilt itself with one op per launch
-    // what build() had chosen before a give-up switched the shared launches off, and when they are tried again: after
-    // rearm_after clean steps (doubled by every further give-up; 0 = never)
-    bool shared_qkv_attn = false, shared_lm_argmax = false, fell_back = false;
-    int rearm_after = 256;
-    long clean_steps = 0;
-    // streaming_kv: the ring inputs of the step in flight (host copies: the operators take them at launch time, as the
-    // reference's kernels do), kv_position on the device, and the operators' [heads, S, D] tensors
-    int ring_sink = 0, ring_window = 0, ring_start = 0, h_past = 0, h_active = 0;
-    int64_t *d_kvpos = nullptr;
-    void *q_ref = nullptr, *k_new = nullptr, *v_new = nullptr, *attn_ref = nullptr, *k_rot = nullptr;
-    void *ring_ws = nullptr;      // ... and the scratch memory of the ring attention (rank-ordered rows, partial results)
-    size_t ring_ws_bytes = 0;
-    int last_status = 0;          // of the last model() call on this state
-    void *warena = nullptr;       // weight_arena: every linear weight and scale of the model in one allocation, in execution order
-    mynn_kv_pages *pages = nullptr;  // kv_page_rows: the session's page table (the caller's); k_cache / v_cache then are pools
-    KvPaging paging;
-    void *ws = nullptr;           // executors that dequantise a weight per call (M >= 16, no resident copy): their own workspace
-    // per-launch record of the last enqueue (names + algorithmic bytes), events when profiling
-    std::vector<Launch> record;
-    bool profiling = false;
-    std::vector<hipEvent_t> events;
-};
 
 static mynn_model_config g_cfg{};
 static bool g_cfg_set = false;
 static std::mutex g_mu;
-
-static size_t align_up(size_t v, size_t a) { return (v + a - 1) / a * a; }
-
-struct ArenaPlan {
-    size_t off = 0;
-    size_t take(size_t bytes) {
-        size_t o = off;
-        off = align_up(off + bytes, 256);
-        return o;
-    }
-};
-
-static void note(Model &m, const char *name, double bytes, double flops = 0.0) {
-    if (m.profiling) {
-        // the launch that follows stamps these two with its own start and end
-        hipEvent_t a, b;
-        hipEventCreate(&a);
-        hipEventCreate(&b);
-        m.events.push_back(a);
-        m.events.push_back(b);
-        launch_timer() = LaunchTimer{a, b};
-    }
-    m.record.push_back({name, bytes, flops});
-}
-
-#define TRY(expr)            \
-    do {                     \
-        int rc__ = (expr);   \
-        if (rc__) return rc__; \
-    } while (0)
 
 // one matrix-core GEMM against a resident dequantised weight
 static int gemm_rows(Model &m, void *out, const void *act, const void *wt, const void *res, int M, int N, int K, int epi,
@@ -615,6 +466,7 @@ static int enqueue_step(Model &m) {
 }
 
 static int enqueue(Model &m) {
+    if (m.net) return enqueue_layered(m);
     return dispatch_dtype16(m.cfg.dtype, [&](auto *t) {
         using T = std::remove_pointer_t<decltype(t)>;
         return enqueue_step<T>(m);
@@ -637,6 +489,18 @@ static int interleave_rows(void **out, const void *a, const void *b, size_t rows
     MYNN_HIP(hipMalloc(out, 2 * rows * row_bytes));
     MYNN_HIP(hipMemcpy2D(*out, 2 * row_bytes, a, row_bytes, row_bytes, rows, hipMemcpyDeviceToDevice));
     MYNN_HIP(hipMemcpy2D((char *)*out + row_bytes, 2 * row_bytes, b, row_bytes, row_bytes, rows, hipMemcpyDeviceToDevice));
+    return 0;
+}
+
+// the page set found in session_state must be one for this batch, these sequences and this page size
+int executor_bind_pages(Model &m) {
+    const mynn_model_config &c = m.cfg;
+    MYNN_REQUIRE(m.pages, MYNN_ERR_INVALID, "model_init: kv_page_rows without a page set after the pools in session_state");
+    m.paging = kv_pages_paging(m.pages);
+    MYNN_REQUIRE((1 << m.paging.shift) == c.kv_page_rows && m.paging.pages_per_seq * c.kv_page_rows == c.max_seq &&
+                     kv_pages_batch(m.pages) == c.batch,
+                 MYNN_ERR_INVALID, "model_init: the page set (batch %d, %d pages of %d rows) does not fit batch %d, max_seq %d, kv_page_rows %d",
+                 kv_pages_batch(m.pages), m.paging.pages_per_seq, 1 << m.paging.shift, c.batch, c.max_seq, c.kv_page_rows);
     return 0;
 }
 
@@ -726,12 +590,7 @@ static int build(Model &m, void **init, void **state) {
     }
     if (c.kv_page_rows) {
         m.pages = (mynn_kv_pages *)state[(c.quant_kv_cache ? 4 : 2) * c.n_layers];
-        MYNN_REQUIRE(m.pages, MYNN_ERR_INVALID, "model_init: kv_page_rows without a page set after the pools in session_state");
-        m.paging = kv_pages_paging(m.pages);
-        MYNN_REQUIRE((1 << m.paging.shift) == c.kv_page_rows && m.paging.pages_per_seq * c.kv_page_rows == c.max_seq &&
-                         kv_pages_batch(m.pages) == c.batch,
-                     MYNN_ERR_INVALID, "model_init: the page set (batch %d, %d pages of %d rows) does not fit batch %d, max_seq %d, kv_page_rows %d",
-                     kv_pages_batch(m.pages), m.paging.pages_per_seq, 1 << m.paging.shift, c.batch, c.max_seq, c.kv_page_rows);
+        TRY(executor_bind_pages(m));
     }
     ws.repacked = true;
     m.final_norm = init[i++];
@@ -1040,6 +899,7 @@ static void destroy(Model *m) {
     if (m->graph_loop_exec) hipGraphExecDestroy(m->graph_loop_exec);
     if (m->graph_loop) hipGraphDestroy(m->graph_loop);
     weight_set_release(m->wset);
+    if (m->net) destroy_layered(*m);
     if (m->ws) hipFree(m->ws);
     if (m->warena) hipFree(m->warena);
     if (m->cos_t) hipFree(m->cos_t);
@@ -1051,31 +911,38 @@ static void destroy(Model *m) {
 }
 
 // H2D of one step's inputs (ids, positions, past_len, active, step counter = 0) in one copy
-static int upload_inputs(Model &m, const int64_t *ids, const int64_t *pos, int64_t past, int64_t active) {
+// n: new tokens per sequence (a layered model takes any number up to seq_q; the Llama graph exactly seq_q)
+static int upload_inputs(Model &m, const int64_t *ids, const int64_t *pos, int64_t past, int64_t active, int n) {
     const mynn_model_config &c = m.cfg;
-    const int rows = c.batch * c.seq_q;
+    const int rows = c.batch * n;
     // (streaming_kv: past_len is the session's unbounded stream position; the ring map folds it into the cache)
-    MYNN_REQUIRE(past >= 0 && (c.streaming_kv ? past + c.seq_q <= INT32_MAX : past + c.seq_q <= c.max_seq), MYNN_ERR_TOO_LONG,
-                 "past_len %lld + %d rows exceeds max_seq %d", (long long)past, c.seq_q, c.max_seq);
+    MYNN_REQUIRE(past >= 0 && (c.streaming_kv ? past + n <= INT32_MAX : past + n <= c.max_seq), MYNN_ERR_TOO_LONG,
+                 "past_len %lld + %d rows exceeds max_seq %d", (long long)past, n, c.max_seq);
     MYNN_REQUIRE(active >= 1 && active <= c.max_seq, MYNN_ERR_INVALID, "active_seq_kv %lld out of range", (long long)active);
     // paged cache: every row the step writes or may read has a page before anything is launched
-    if (m.pages) TRY(kv_pages_reserve(m.pages, std::max<long>(past + c.seq_q, active)));
-    for (int s = 0; s < c.seq_q; s++)
+    if (m.pages) TRY(kv_pages_reserve(m.pages, std::max<long>(past + n, active)));
+    for (int s = 0; s < n; s++)
         MYNN_REQUIRE(pos[s] >= 0 && pos[s] < c.max_seq, MYNN_ERR_INVALID, "position_id[%d]=%lld outside the RoPE table", s,
                      (long long)pos[s]);
+    if (m.net) {  // its positions follow from past_len
+        for (int s = 0; s < n; s++)
+            MYNN_REQUIRE(pos[s] == past + s, MYNN_ERR_INVALID, "position_id[%d]=%lld after %lld tokens", s, (long long)pos[s], (long long)past);
+        MYNN_REQUIRE(active == past + n, MYNN_ERR_INVALID, "active_seq_kv %lld after %lld + %d tokens", (long long)active, (long long)past, n);
+    }
+    m.rows_now = n;
     for (int r = 0; r < rows; r++)
         MYNN_REQUIRE(ids[r] >= -c.vocab && ids[r] < c.vocab, MYNN_ERR_INVALID, "input_ids[%d]=%lld outside the vocabulary", r,
                      (long long)ids[r]);
     int64_t *h_ids = (int64_t *)m.h_stage;
     int64_t *h_pos = h_ids + rows;
-    int32_t *h_sc = (int32_t *)(h_pos + c.seq_q);
+    int32_t *h_sc = (int32_t *)(h_pos + n);
     memcpy(h_ids, ids, (size_t)rows * 8);
-    memcpy(h_pos, pos, (size_t)c.seq_q * 8);
+    memcpy(h_pos, pos, (size_t)n * 8);
     h_sc[0] = (int32_t)past; h_sc[1] = (int32_t)active; h_sc[2] = 0;
     m.h_past = (int)past;
     m.h_active = (int)active;
     MYNN_HIP(hipMemcpyAsync(m.d_ids, h_ids, (size_t)rows * 8, hipMemcpyHostToDevice, m.stream));
-    MYNN_HIP(hipMemcpyAsync(m.d_pos, h_pos, (size_t)c.seq_q * 8, hipMemcpyHostToDevice, m.stream));
+    MYNN_HIP(hipMemcpyAsync(m.d_pos, h_pos, (size_t)n * 8, hipMemcpyHostToDevice, m.stream));
     MYNN_HIP(hipMemcpyAsync(m.d_past, h_sc, 12, hipMemcpyHostToDevice, m.stream));
     return 0;
 }
@@ -1126,8 +993,10 @@ static int handover_clean_steps(Model &m, long steps) {
     return capture_step(m);
 }
 
+bool model_takes_any_rows(const void *state) { return state && ((const Model *)state)->net != nullptr; }
+
 static int run_once(Model &m) {
-    if (m.use_graph && !m.profiling) {
+    if (m.use_graph && !m.profiling && m.sel_count == m.cfg.batch) {  // (the captured step makes every sequence's logits)
         MYNN_HIP(hipGraphLaunch(m.graph_exec, m.stream));
         return 0;
     }
@@ -1138,8 +1007,30 @@ static int run_once(Model &m) {
 
 using namespace mynn;
 
+static void select_all(Model &m, int n) {
+    m.sel_first = 0;
+    m.sel_stride = 1;
+    m.sel_count = m.cfg.batch * n;
+}
+
+static int check_layered_config(const mynn_model_config *cfg) {
+    auto spec = arch_spec(cfg->arch);
+    MYNN_REQUIRE(spec && spec->family == ModelSpec::LAYERED, MYNN_ERR_INVALID, "model_configure: no layered architecture %d", cfg->arch);
+    MYNN_REQUIRE(cfg->dtype == MYNN_BF16 || cfg->dtype == MYNN_F32, MYNN_ERR_UNSUPPORTED, "model_configure: %s runs in bf16 or f32 (dtype %d)",
+                 spec->architecture.c_str(), cfg->dtype);
+    MYNN_REQUIRE(cfg->max_seq > 0 && cfg->seq_q > 0 && cfg->batch > 0 && cfg->seq_q <= cfg->max_seq, MYNN_ERR_INVALID,
+                 "model_configure: max_seq %d, seq_q %d, batch %d", cfg->max_seq, cfg->seq_q, cfg->batch);
+    MYNN_REQUIRE(!cfg->weights_int8 && !cfg->quant_kv_cache && !cfg->quantize_activations && !cfg->streaming_kv && !cfg->qkv_bias && !cfg->weight_arena,
+                 MYNN_ERR_UNSUPPORTED, "model_configure: %s takes none of the Llama graph's options", spec->architecture.c_str());
+    const int P = cfg->kv_page_rows;
+    MYNN_REQUIRE(!P || (P >= 64 && (P & (P - 1)) == 0 && cfg->max_seq % P == 0), MYNN_ERR_INVALID,
+                 "model_configure: kv_page_rows %d (a power of two >= 64 that divides max_seq %d)", P, cfg->max_seq);
+    return 0;
+}
+
 static int check_config(const mynn_model_config *cfg) {
     MYNN_REQUIRE(cfg, MYNN_ERR_INVALID, "model_configure: null config");
+    if (cfg->arch) return check_layered_config(cfg);
     MYNN_REQUIRE(cfg->n_layers > 0 && cfg->hidden > 0 && cfg->n_heads > 0 && cfg->n_kv_heads > 0 && cfg->head_dim > 0 &&
                      cfg->ffn > 0 && cfg->vocab > 0 && cfg->max_seq > 0 && cfg->seq_q > 0 && cfg->batch > 0,
                  MYNN_ERR_INVALID, "model_configure: non-positive dimension");
@@ -1184,8 +1075,11 @@ static void *model_create_with(const mynn_model_config *cfg, WeightSet *wset, vo
     Model *m = new Model;
     m->cfg = *cfg;
     m->quant = cfg->weights_int8 != 0;
+    m->logits_dtype = cfg->arch ? MYNN_F32 : cfg->dtype;
+    m->rows_now = cfg->seq_q;
+    select_all(*m, cfg->seq_q);
     m->wset = wset;  // (one reference is the model's from here on: destroy() lets it go)
-    if (build(*m, wset->initializer.data(), session_state)) {
+    if (cfg->arch ? build_layered(*m, session_state) || capture_step(*m) : build(*m, wset->initializer.data(), session_state)) {
         destroy(m);
         return nullptr;
     }
@@ -1269,7 +1163,8 @@ extern "C" void free_pinned(void *p) {
 static int step_once(Model &m, const int64_t *input_ids, const int64_t *position_id, int64_t past_len, int64_t active_seq_kv,
                      int32_t *next_token, void *logits_host, bool *handover_failed) {
     *handover_failed = false;
-    TRY(upload_inputs(m, input_ids, position_id, past_len, active_seq_kv));
+    select_all(m, m.cfg.seq_q);
+    TRY(upload_inputs(m, input_ids, position_id, past_len, active_seq_kv, m.cfg.seq_q));
     TRY(run_once(m));
     const mynn_model_config &c = m.cfg;
     char *h_next = m.h_stage + m.stage_bytes - m.next_stage;
@@ -1277,7 +1172,7 @@ static int step_once(Model &m, const int64_t *input_ids, const int64_t *position
     if (m.qkv_attn) MYNN_HIP(hipMemcpyAsync(h_next, m.d_past + 3, 24, hipMemcpyDeviceToHost, m.stream));
     else if (next_token) MYNN_HIP(hipMemcpyAsync(h_next, m.d_next, (size_t)c.batch * 4, hipMemcpyDeviceToHost, m.stream));
     if (logits_host)
-        MYNN_HIP(hipMemcpyAsync(logits_host, m.logits, (size_t)c.batch * c.seq_q * c.vocab * dtype_size(c.dtype),
+        MYNN_HIP(hipMemcpyAsync(logits_host, m.logits, (size_t)c.batch * c.seq_q * c.vocab * dtype_size(m.logits_dtype),
                                 hipMemcpyDeviceToHost, m.stream));
     MYNN_HIP(hipStreamSynchronize(m.stream));
     if (m.qkv_attn) {
@@ -1303,6 +1198,54 @@ extern "C" int mynn_model_step(void *state, const int64_t *input_ids, const int6
     TRY(handover_recover(m));
     TRY(step_once(m, input_ids, position_id, past_len, active_seq_kv, next_token, logits_host, &failed));
     return failed ? fail(MYNN_ERR_STATE, "decode step: hand-over failure after recovery") : 0;
+}
+
+// `rows` new tokens per sequence, logits of some of them as f32
+extern "C" int mynn_model_step_rows(void *state, const int64_t *input_ids, int rows, int64_t past_len, int logit_first, int logit_rows,
+                                    int32_t *next_token, float *logits_host) {
+    MYNN_REQUIRE(state && input_ids, MYNN_ERR_INVALID, "model_step_rows: null argument");
+    Model &m = *(Model *)state;
+    const mynn_model_config &c = m.cfg;
+    MYNN_REQUIRE(rows >= 1 && rows <= c.seq_q && !c.streaming_kv, MYNN_ERR_INVALID, "model_step_rows: %d rows (seq_q %d)", rows, c.seq_q);
+    MYNN_REQUIRE(logit_first >= 0 && logit_rows >= 0 && logit_first + logit_rows <= rows, MYNN_ERR_INVALID,
+                 "model_step_rows: logits of rows %d .. %d of %d", logit_first, logit_first + logit_rows, rows);
+    MYNN_REQUIRE(c.batch == 1 || ((logit_rows == 0 || logit_rows == rows || (logit_rows == 1 && logit_first == rows - 1)) && (m.net || rows == c.seq_q)),
+                 MYNN_ERR_UNSUPPORTED, "model_step_rows: a batch takes no, the last or all logits%s", m.net ? "" : " and whole steps");
+    MYNN_REQUIRE(!next_token || logit_first + logit_rows == rows && logit_rows > 0, MYNN_ERR_INVALID, "model_step_rows: the next token needs the last row's logits");
+    const int B = c.batch, V = c.vocab;
+    if (!m.net) {
+        // the Llama graph: always seq_q rows and all their logits; a short portion is zero-padded
+        std::vector<int64_t> ids((size_t)B * c.seq_q, 0), pos(c.seq_q);
+        for (int b = 0; b < B; b++) memcpy(&ids[(size_t)b * c.seq_q], input_ids + (size_t)b * rows, (size_t)rows * 8);
+        for (int s = 0; s < c.seq_q; s++) pos[s] = past_len + s;
+        TRY(mynn_model_step(state, ids.data(), pos.data(), past_len, past_len + c.seq_q, rows == c.seq_q ? next_token : nullptr, nullptr));
+        if (next_token && rows < c.seq_q) TRY(mynn_model_argmax_row(state, rows - 1, next_token));
+        if (logits_host && logit_rows) {
+            std::vector<uint16_t> h((size_t)logit_rows * V);
+            for (int b = 0; b < B; b++) {
+                MYNN_HIP(hipMemcpy(h.data(), (const uint16_t *)m.logits + ((size_t)b * c.seq_q + logit_first) * V, h.size() * 2, hipMemcpyDeviceToHost));
+                float *dst = logits_host + (size_t)b * logit_rows * V;
+                for (size_t i = 0; i < h.size(); i++)
+                    dst[i] = c.dtype == MYNN_BF16 ? bf16_bits_to_f32(h[i]) : (float)__builtin_bit_cast(f16_t, h[i]);
+            }
+        }
+        return 0;
+    }
+    std::vector<int64_t> pos(rows);
+    for (int s = 0; s < rows; s++) pos[s] = past_len + s;
+    m.sel_count = B * logit_rows;
+    m.sel_first = logit_first;
+    m.sel_stride = B > 1 && logit_rows == 1 ? rows : 1;
+    if (c.seq_q == 1) select_all(m, 1);  // (the captured step makes them anyway)
+    TRY(upload_inputs(m, input_ids, pos.data(), past_len, past_len + rows, rows));
+    TRY(run_once(m));
+    char *h_next = m.h_stage + m.stage_bytes - m.next_stage;
+    if (next_token) MYNN_HIP(hipMemcpyAsync(h_next, m.d_next, (size_t)B * 4, hipMemcpyDeviceToHost, m.stream));
+    if (logits_host && logit_rows)
+        MYNN_HIP(hipMemcpyAsync(logits_host, m.logits, (size_t)B * logit_rows * V * 4, hipMemcpyDeviceToHost, m.stream));
+    MYNN_HIP(hipStreamSynchronize(m.stream));
+    if (next_token) memcpy(next_token, h_next, (size_t)B * 4);
+    return 0;
 }
 
 extern "C" int mynn_model_step_streaming(void *state, const int64_t *input_ids, const int64_t *position_id, int64_t past_len,
@@ -1373,15 +1316,16 @@ extern "C" int mynn_model_argmax_row(void *state, int row, int32_t *token) {
     MYNN_REQUIRE(state && token, MYNN_ERR_INVALID, "model_argmax_row: null argument");
     Model &m = *(Model *)state;
     const mynn_model_config &c = m.cfg;
-    MYNN_REQUIRE(row >= 0 && row < c.batch * c.seq_q, MYNN_ERR_INVALID, "model_argmax_row: row %d", row);
-    const char *l = (const char *)m.logits + (size_t)row * c.vocab * dtype_size(c.dtype);
-    TRY(mynn_argmax_last(m.d_next, l, c.vocab, c.dtype, m.stream));
+    MYNN_REQUIRE(row >= 0 && row < (m.net ? m.sel_count : c.batch * c.seq_q), MYNN_ERR_INVALID, "model_argmax_row: row %d", row);
+    const char *l = (const char *)m.logits + (size_t)row * c.vocab * dtype_size(m.logits_dtype);
+    TRY(mynn_argmax_last(m.d_next, l, c.vocab, m.logits_dtype, m.stream));
     MYNN_HIP(hipMemcpyAsync(m.h_stage, m.d_next, 4, hipMemcpyDeviceToHost, m.stream));
     MYNN_HIP(hipStreamSynchronize(m.stream));
     memcpy(token, m.h_stage, 4);
     return 0;
 }
 
+extern "C" int mynn_model_vocab(void *state) { return state ? ((Model *)state)->cfg.vocab : MYNN_ERR_INVALID; }
 extern "C" const void *mynn_model_logits_device(void *state) { return state ? ((Model *)state)->logits : nullptr; }
 
 extern "C" int mynn_model_stats(void *state, size_t *arena_bytes, int *launches_per_step, int *graph) {
@@ -1400,10 +1344,11 @@ extern "C" int mynn_model_decode_loop(void *state, int32_t token, int64_t past_l
     MYNN_REQUIRE(c.batch * c.seq_q == 1 && !c.streaming_kv, MYNN_ERR_STATE, "decode_loop: needs a batch-1 decode model without streaming_kv");
     MYNN_REQUIRE(past_len + n_steps <= c.max_seq && n_steps <= m.token_cap, MYNN_ERR_TOO_LONG,
                  "decode_loop: past_len %lld + %d steps exceeds max_seq %d", (long long)past_len, n_steps, c.max_seq);
+    select_all(m, 1);
     if (m.pages) TRY(kv_pages_reserve(m.pages, past_len + n_steps));
     for (int attempt = 0; attempt < 2; attempt++) {
         int64_t id = token, pos = past_len;
-        TRY(upload_inputs(m, &id, &pos, past_len, past_len + 1));
+        TRY(upload_inputs(m, &id, &pos, past_len, past_len + 1, 1));
         int done = 0;
         if (m.use_graph && !m.profiling && m.graph_loop_exec)
             for (; done + kLoopSteps <= n_steps; done += kLoopSteps) MYNN_HIP(hipGraphLaunch(m.graph_loop_exec, m.stream));
@@ -1425,6 +1370,7 @@ extern "C" int mynn_model_decode_loop(void *state, int32_t token, int64_t past_l
 }
 
 static int profile_enqueue(Model &m, mynn_kernel_time *out, int cap) {
+    select_all(m, m.rows_now);
     for (hipEvent_t e : m.events) hipEventDestroy(e);
     m.events.clear();
     m.profiling = true;
@@ -1455,7 +1401,7 @@ extern "C" int mynn_model_profile_step(void *state, int32_t token, int64_t past_
     const mynn_model_config &c = m.cfg;
     MYNN_REQUIRE(c.batch * c.seq_q == 1, MYNN_ERR_STATE, "profile_step: needs a batch-1 decode model");
     int64_t id = token, pos = past_len;
-    TRY(upload_inputs(m, &id, &pos, past_len, past_len + 1));
+    TRY(upload_inputs(m, &id, &pos, past_len, past_len + 1, 1));
     return profile_enqueue(m, out, cap);
 }
 
@@ -1463,6 +1409,6 @@ extern "C" int mynn_model_profile(void *state, const int64_t *input_ids, const i
                                   int64_t active_seq_kv, mynn_kernel_time *out, int cap) {
     MYNN_REQUIRE(state && input_ids && position_id && out && cap > 0, MYNN_ERR_INVALID, "profile: bad argument");
     Model &m = *(Model *)state;
-    TRY(upload_inputs(m, input_ids, position_id, past_len, active_seq_kv));
+    TRY(upload_inputs(m, input_ids, position_id, past_len, active_seq_kv, m.cfg.seq_q));
     return profile_enqueue(m, out, cap);
 }

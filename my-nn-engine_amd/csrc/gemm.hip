@@ -18,6 +18,7 @@
 #include <mutex>
 
 #include "kernels.h"
+#include "dense_load.h"
 #include "mfma.h"
 
 namespace mynn {
@@ -100,11 +101,37 @@ __device__ __forceinline__ void gemm_store(AccAt at, uint16_t *lds, T *C, const 
                                            int n0, int wrow, int wcol, int lane, int wave) {
     constexpr int TI = G::TI, TJ = G::TJ;
     constexpr int EST = G::EST;
-    static_assert(EPI != GEMM_SWIGLU || TJ % 2 == 0, "the SwiGLU store pairs neighbouring column tiles");
-    constexpr int OC = EPI == GEMM_SWIGLU ? TJ * 16 : TJ * 32;  // output columns of the wave tile
-    constexpr int CPR = OC / 8;                                 // 16-byte chunks per strip row
-    const int ldc = EPI == GEMM_SWIGLU ? N >> 1 : N;
-    const int c0 = EPI == GEMM_SWIGLU ? (n0 + wcol) >> 1 : n0 + wcol;
+    constexpr bool GATED = EPI == GEMM_SWIGLU || EPI == GEMM_GEGLU;
+    static_assert(!GATED || TJ % 2 == 0, "the gated stores pair neighbouring column tiles");
+    if constexpr (EPI == GEMM_F32) {
+        // f32 straight from the accumulators: four neighbouring columns of a row per lane
+        float *F = (float *)C;
+        const float sc = R ? *(const float *)R : 1.f;
+        const bool vec4 = (N & 3) == 0;
+#pragma unroll
+        for (int i = 0; i < TI; i++) {
+            const int row = m0 + wrow + i * 32 + (lane & 31);
+            if (row >= M) continue;
+#pragma unroll
+            for (int j = 0; j < TJ; j++)
+#pragma unroll
+                for (int q = 0; q < 4; q++) {
+                    const int col = n0 + wcol + j * 32 + 8 * q + 4 * (lane >> 5);
+                    float *dst = F + (size_t)row * N + col;
+                    const float4 v = float4{at(i, j, 4 * q) * sc, at(i, j, 4 * q + 1) * sc, at(i, j, 4 * q + 2) * sc, at(i, j, 4 * q + 3) * sc};
+                    if (vec4 && col + 4 <= N) *(float4 *)dst = v;
+                    else {
+                        const float f[4] = {v.x, v.y, v.z, v.w};
+                        for (int x = 0; x < 4 && col + x < N; x++) dst[x] = f[x];
+                    }
+                }
+        }
+        return;
+    }
+    constexpr int OC = GATED ? TJ * 16 : TJ * 32;  // output columns of the wave tile
+    constexpr int CPR = OC / 8;                    // 16-byte chunks per strip row
+    const int ldc = GATED ? N >> 1 : N;
+    const int c0 = GATED ? (n0 + wcol) >> 1 : n0 + wcol;
     T *patch = (T *)lds + (size_t)wave * 32 * EST;
     const bool vec_ok = (ldc & 7) == 0;
 #pragma unroll
@@ -112,7 +139,19 @@ __device__ __forceinline__ void gemm_store(AccAt at, uint16_t *lds, T *C, const 
         T *prow = patch + (lane & 31) * EST + (lane >> 5) * 4;
 #pragma unroll
         for (int q = 0; q < 4; q++) {
-            if (EPI == GEMM_SWIGLU) {
+            if constexpr (EPI == GEMM_GEGLU) {
+                // (gate and up enter the activation as the f32 sums they are)
+#pragma unroll
+                for (int j = 0; j < TJ; j += 2) {
+                    float o[4];
+#pragma unroll
+                    for (int x = 0; x < 4; x++) {
+                        const float g = at(i, j, 4 * q + x), u = at(i, j + 1, 4 * q + x);
+                        o[x] = g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(gelu_tanh_arg(g) * -1.4426950408889634f)) * u;
+                    }
+                    *(uint2 *)(prow + j * 16 + 8 * q) = uint2{pack2<T>(o[0], o[1]), pack2<T>(o[2], o[3])};
+                }
+            } else if constexpr (EPI == GEMM_SWIGLU) {
 #pragma unroll
                 for (int j = 0; j < TJ; j += 2) {
                     float o[4];
@@ -166,7 +205,8 @@ __device__ __forceinline__ void gemm_store(AccAt at, uint16_t *lds, T *C, const 
 // KTAIL: K is not a multiple of 2*BK, so the last steps mask the columns of A past K.
 // EPI: GEMM_PLAIN C = T(acc); GEMM_RESIDUAL C = T(R + T(acc)) with R laid out like C;
 // GEMM_SWIGLU: B's rows are gate/up interleaved in groups of 32, C is [M, N/2] and
-// C = T(swish(T(acc_gate)) * T(acc_up)) -- the roundings of separate linear, Add and SwiGLU ops.
+// C = T(swish(T(acc_gate)) * T(acc_up)) -- the roundings of separate linear, Add and SwiGLU ops;
+// GEMM_GEGLU: the same rows, C = T(gelu_tanh(acc_gate) * acc_up); GEMM_F32: C is f32 [M, N], times *(float *)R when given.
 template <typename T, typename G, bool KTAIL, int EPI>
 __global__ __launch_bounds__(G::THREADS) void gemm_nt_mfma_kernel(T *C, const T *A, const T *B, const T *R, int M, int N,
                                                                  int K, int Kp) {
@@ -553,7 +593,7 @@ static int gemm_launch(void *out, const void *act, const void *wt, const void *r
     // the direct-to-LDS kernel is the faster 256 x 256 one (measured +5..20%); it needs whole 64-wide K steps
     const bool dma_ok = K % 64 == 0 && g_gemm_tile_override != 2;
     if (g_gemm_tile_override == 3 || g_gemm_tile_override == 4) big = dma_ok;
-    if constexpr (EPI != GEMM_SWIGLU) {
+    if constexpr (EPI != GEMM_SWIGLU && EPI != GEMM_GEGLU) {
         // 320 columns per tile when that saves rounds over the CUs (rounds x tile width = time)
         const long wide_tiles = (long)((M + 255) / 256) * ((N + 319) / 320);
         const long cost256 = (big_tiles + 255) / 256 * 256, cost320 = (wide_tiles + 255) / 256 * 320;
@@ -573,9 +613,14 @@ int gemm_nt_mfma(void *out, const void *act, const void *wt, const void *res, in
     MYNN_REQUIRE(M > 0 && N > 0 && K > 0 && K % 8 == 0, MYNN_ERR_INVALID, "dequant_matmul: M=%d N=%d K=%d", M, N, K);
     MYNN_REQUIRE(aligned16(act) && aligned16(wt), MYNN_ERR_INVALID, "dequant_matmul: act must be 16-byte aligned");
     MYNN_REQUIRE(epi != GEMM_RESIDUAL || res, MYNN_ERR_INVALID, "dequant_matmul: residual store without a residual");
-    MYNN_REQUIRE(epi != GEMM_SWIGLU || N % 64 == 0, MYNN_ERR_INVALID, "dequant_matmul: SwiGLU store needs N %% 64 == 0, N=%d", N);
+    MYNN_REQUIRE((epi != GEMM_SWIGLU && epi != GEMM_GEGLU) || N % 64 == 0, MYNN_ERR_INVALID, "dequant_matmul: a gated store needs N %% 64 == 0, N=%d", N);
     return dispatch_dtype16(dtype, [&](auto *t) {
         using T = std::remove_pointer_t<decltype(t)>;
+        if constexpr (std::is_same<T, bf16_t>::value) {
+            if (epi == GEMM_GEGLU) return gemm_launch<T, GEMM_GEGLU>(out, act, wt, res, M, N, K, tile, s);
+            if (epi == GEMM_F32) return gemm_launch<T, GEMM_F32>(out, act, wt, res, M, N, K, tile, s);
+        }
+        MYNN_REQUIRE(epi <= GEMM_SWIGLU, MYNN_ERR_UNSUPPORTED, "dequant_matmul: store %d is built for bf16", epi);
         if (epi == GEMM_RESIDUAL) return gemm_launch<T, GEMM_RESIDUAL>(out, act, wt, res, M, N, K, tile, s);
         if (epi == GEMM_SWIGLU) return gemm_launch<T, GEMM_SWIGLU>(out, act, wt, res, M, N, K, tile, s);
         return gemm_launch<T, GEMM_PLAIN>(out, act, wt, res, M, N, K, tile, s);

@@ -59,7 +59,8 @@ int dequant_gemm_skinny(void *out, const void *act, const int8_t *wq, bool packe
 // matrix-core GEMM pieces.  A dequantised weight is [N, Kp] of the 16-bit type, Kp = K rounded up to 64,
 // zero padded (gemm_weight_bytes); dequant_weight_rows writes one (group/which: see gemm.hip), and
 // gemm_nt_mfma multiplies by it: out = store(act . wt^T) with the store one of GEMM_*.
-enum { GEMM_PLAIN = 0, GEMM_RESIDUAL = 1, GEMM_SWIGLU = 2 };
+// GEMM_GEGLU, GEMM_F32: bf16 operands (store forms of executors with a 32-bit residual stream; see gemm.hip).
+enum { GEMM_PLAIN = 0, GEMM_RESIDUAL = 1, GEMM_SWIGLU = 2, GEMM_GEGLU = 3, GEMM_F32 = 4 };
 size_t gemm_weight_bytes(int N, int K);
 int dequant_weight_rows(void *dst, const int8_t *wq, const void *scale, int N, int K, int dtype, int group, int which,
                         hipStream_t s);

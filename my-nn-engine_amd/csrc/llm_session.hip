@@ -6,7 +6,8 @@
 #include <cstring>
 #include <vector>
 
-#include "mynn_common.h"
+#include "executor.h"
+#include "session.h"
 
 using namespace mynn;
 
@@ -65,17 +66,6 @@ extern "C" int mynn_rope_table(void *cos_t, void *sin_t, int max_seq, int head_d
 }
 
 // ---- LlmSession -------------------------------------------------------------------------------
-struct mynn_llm {
-    void *decode = nullptr, *prefill = nullptr;
-    int prefill_len = 0, max_seq = 0;
-    int64_t eos = -1, past_len = 0;
-    mynn_step_fn step = nullptr;
-    void *user = nullptr;
-    int last_error = 0;
-    bool streaming = false;  // DecodeKind::LlamaStreaming { sink, window }
-    int sink = 0, window = 0;
-};
-
 // streaming_kv_position (session.rs:604-635): the recency rank of every cache slot -- sink slots keep their position,
 // ring slots are walked in age order from ring_start, slots not written yet keep their own index
 static void streaming_kv_position(std::vector<int64_t> &out, int64_t sink, int64_t window, int64_t stream_pos) {
@@ -130,7 +120,12 @@ extern "C" mynn_llm *mynn_llm_create_with_step(mynn_step_fn step, void *user, in
     l->eos = eos_token_id;
     return l;
 }
-extern "C" void mynn_llm_destroy(mynn_llm *l) { delete l; }
+extern "C" void mynn_llm_destroy(mynn_llm *l) {
+    if (l && l->release) l->release(l);
+    delete l;
+}
+extern "C" void *mynn_llm_decode_state(mynn_llm *l) { return l ? l->decode : nullptr; }
+extern "C" void *mynn_llm_prefill_state(mynn_llm *l) { return l ? l->prefill : nullptr; }
 // reset (session.rs:303-305): past_len = 0; a paged cache also gives its pages back to the pool (the prefill model shares
 // the decode model's page set)
 extern "C" void mynn_llm_reset(mynn_llm *l) {
@@ -180,6 +175,16 @@ static int run_prefill(mynn_llm *l, const int64_t *ids, size_t n, int64_t *next)
             pos[i] = l->past_len + (int64_t)i;
         }
         int32_t t = 0;
+        if (model_takes_any_rows(l->prefill)) {  // no padding: the portion as it is, logits of its last row at most
+            const bool end = chunk == n;
+            int rc = mynn_model_step_rows(l->prefill, ids, (int)chunk, l->past_len, (int)chunk - 1, end ? 1 : 0, end ? &t : nullptr, nullptr);
+            if (rc) return rc;
+            l->past_len += (int64_t)chunk;
+            if (end) *next = t;
+            ids += chunk;
+            n -= chunk;
+            continue;
+        }
         // the token wanted is that of row chunk-1; the model reports the last row, so the final
         // (possibly padded) chunk reads its logits back
         const bool last = chunk == n;
@@ -212,13 +217,47 @@ static int run_prefill(mynn_llm *l, const int64_t *ids, size_t n, int64_t *next)
     return 0;
 }
 
+// Portions of at most prefill_len tokens through the prefill model, single tokens through the decode model.
+extern "C" int mynn_llm_feed(mynn_llm *l, const int64_t *ids, size_t n, const int64_t *want, size_t n_want, float *logits) {
+    MYNN_REQUIRE(l && !l->step && !l->streaming && (ids || n == 0) && ((want && logits) || n_want == 0), MYNN_ERR_INVALID, "llm_feed: bad argument");
+    for (size_t i = 0; i < n_want; i++)
+        MYNN_REQUIRE(want[i] >= (i ? want[i - 1] + 1 : 0) && want[i] < (int64_t)n, MYNN_ERR_INVALID, "llm_feed: want[%zu] = %lld of %zu tokens", i,
+                     (long long)want[i], n);
+    MYNN_REQUIRE(l->past_len + (int64_t)n <= l->max_seq, MYNN_ERR_TOO_LONG, "llm_feed: %lld + %zu tokens exceed max_seq %d", (long long)l->past_len, n,
+                 l->max_seq);
+    const int V = mynn_model_vocab(l->decode);
+    std::vector<float> span;
+    size_t w = 0;
+    for (size_t at = 0; at < n;) {
+        // (a Llama prefill model pads its portion to prefill_len rows: they must fit the cache)
+        const bool prefill = l->prefill && n - at > 1 && (model_takes_any_rows(l->prefill) || l->past_len + l->prefill_len <= l->max_seq);
+        void *model = prefill ? l->prefill : l->decode;
+        const size_t chunk = prefill ? std::min<size_t>(n - at, (size_t)l->prefill_len) : 1;
+        size_t w1 = w;
+        while (w1 < n_want && want[w1] < (int64_t)(at + chunk)) w1++;
+        // logits of the rows from the first to the last one asked for in this portion
+        const int first = w1 > w ? (int)(want[w] - (int64_t)at) : 0, rows = w1 > w ? (int)(want[w1 - 1] - want[w]) + 1 : 0;
+        const bool dense = (size_t)rows == w1 - w;  // every row of the span was asked for: straight into the caller's buffer
+        if (!dense) span.resize((size_t)rows * V);
+        float *dst = dense ? logits + w * V : span.data();
+        int rc = mynn_model_step_rows(model, ids + at, (int)chunk, l->past_len, first, rows, nullptr, rows ? dst : nullptr);
+        if (rc) return rc;
+        for (size_t i = w; !dense && i < w1; i++)
+            std::copy_n(span.data() + (size_t)(want[i] - want[w]) * V, V, logits + i * V);
+        w = w1;
+        at += chunk;
+        l->past_len += (int64_t)chunk;
+    }
+    return 0;
+}
+
 extern "C" int mynn_llm_generate_ids(mynn_llm *l, const int64_t *prompt_ids, size_t n_prompt, size_t max_new_tokens,
                                      int64_t *out) {
     MYNN_REQUIRE(l && (prompt_ids || n_prompt == 0) && (out || max_new_tokens == 0), MYNN_ERR_INVALID,
                  "llm_generate_ids: null argument");
     if (n_prompt == 0) return 0;
     const bool prefill_runs = l->prefill != nullptr;
-    const int64_t needed = prefill_runs
+    const int64_t needed = prefill_runs && !model_takes_any_rows(l->prefill)
         ? l->past_len + (int64_t)((n_prompt + l->prefill_len - 1) / l->prefill_len * l->prefill_len)
         : l->past_len + (int64_t)n_prompt;
     MYNN_REQUIRE(l->streaming || l->max_seq >= needed, MYNN_ERR_TOO_LONG, "prompt needs %lld cache rows, max_seq_len is %d (past_len %lld)",

@@ -15,135 +15,11 @@
 #include <string>
 #include <vector>
 
+#include "json.h"
+#include "model_spec.h"
 #include "mynn_common.h"
 
 namespace mynn {
-
-// ---- a JSON reader just large enough for a safetensors header and model.safetensors.index.json ----
-struct Json {
-    enum Kind { NUL, NUM, STR, ARR, OBJ, BOOL } kind = NUL;
-    double num = 0;
-    std::string str;
-    std::vector<Json> arr;
-    std::vector<std::pair<std::string, Json>> obj;  // insertion order
-    const Json *get(const char *key) const {
-        for (auto &kv : obj)
-            if (kv.first == key) return &kv.second;
-        return nullptr;
-    }
-};
-struct JsonParser {
-    const char *p, *end;  // [p, end) is followed by a NUL (parse_json copies the text), so strtod cannot run past it
-    bool ok = true;
-    int depth = 0;
-    static constexpr int kMaxDepth = 32;  // a safetensors header nests 3 deep
-    void ws() {
-        while (p < end && (*p == ' ' || *p == '\n' || *p == '\t' || *p == '\r')) p++;
-    }
-    bool eat(char c) {
-        ws();
-        if (p < end && *p == c) {
-            p++;
-            return true;
-        }
-        return false;
-    }
-    std::string string() {
-        std::string s;
-        if (!eat('"')) {
-            ok = false;
-            return s;
-        }
-        while (p < end && *p != '"') {
-            if (*p == '\\' && p + 1 < end) {
-                p++;
-                switch (*p) {
-                case 'n': s += '\n'; break;
-                case 't': s += '\t'; break;
-                case 'u':  // tensor names are ASCII; keep the escape verbatim
-                    s += "\\u";
-                    break;
-                default: s += *p;
-                }
-                p++;
-            } else s += *p++;
-        }
-        if (p >= end) ok = false;
-        else p++;
-        return s;
-    }
-    Json value() {
-        Json j;
-        ws();
-        if (p >= end) {
-            ok = false;
-            return j;
-        }
-        if ((*p == '{' || *p == '[') && ++depth > kMaxDepth) {
-            ok = false;
-            return j;
-        }
-        if (*p == '{') {
-            p++;
-            j.kind = Json::OBJ;
-            if (eat('}')) {
-                depth--;
-                return j;
-            }
-            do {
-                std::string k = string();
-                if (!ok || !eat(':')) {
-                    ok = false;
-                    return j;
-                }
-                j.obj.emplace_back(std::move(k), value());
-                if (!ok) return j;
-            } while (eat(','));
-            if (!eat('}')) ok = false;
-            depth--;
-        } else if (*p == '[') {
-            p++;
-            j.kind = Json::ARR;
-            if (eat(']')) {
-                depth--;
-                return j;
-            }
-            do {
-                j.arr.push_back(value());
-                if (!ok) return j;
-            } while (eat(','));
-            if (!eat(']')) ok = false;
-            depth--;
-        } else if (*p == '"') {
-            j.kind = Json::STR;
-            j.str = string();
-        } else if ((end - p >= 4 && (!strncmp(p, "true", 4) || !strncmp(p, "null", 4))) || (end - p >= 5 && !strncmp(p, "false", 5))) {
-            j.kind = *p == 'n' ? Json::NUL : Json::BOOL;
-            j.num = *p == 't';
-            p += *p == 'f' ? 5 : 4;
-        } else {
-            char *q = nullptr;
-            j.kind = Json::NUM;
-            j.num = strtod(p, &q);
-            if (q == p || q > end) ok = false;
-            p = q;
-        }
-        return j;
-    }
-};
-static bool parse_json(const char *data, size_t n, Json &out) {
-    const std::string text(data, n);  // NUL-terminated copy: the mapped header may end exactly at the end of the file
-    JsonParser ps{text.c_str(), text.c_str() + n};
-    out = ps.value();
-    return ps.ok;
-}
-
-// a JSON number that must be a non-negative integer below 2^53 (offsets, extents): false otherwise
-static bool as_size(const Json &j, size_t *out) {
-    if (j.kind != Json::NUM || !(j.num >= 0.0) || j.num > 9007199254740992.0 || j.num != (double)(uint64_t)j.num) return false;
-    *out = (size_t)j.num;
-    return true;
-}
 
 // ---- shards ---------------------------------------------------------------------------------------
 struct Shard {
@@ -491,10 +367,45 @@ static int upload_linear(mynn_device_weights &dw, const mynn_weights &w, const s
     return upload_float(dw, w, name + ".scale", dt, N);
 }
 
+// a layered architecture: its tensors in its own order and shapes, in cfg.dtype
+static int upload_arch(mynn_device_weights &dw, const mynn_weights &w, const ModelSpec &spec, int dt) {
+    for (const TensorSpec &t : spec.tensors) {
+        auto it = w.entries.find(t.name);
+        MYNN_REQUIRE(it != w.entries.end(), MYNN_ERR_INVALID, "weights: no tensor named %s", t.name.c_str());
+        MYNN_REQUIRE(it->second.shape == t.shape, MYNN_ERR_INVALID, "weights: %s has another shape than the config gives it", t.name.c_str());
+        if (dt != MYNN_F32) {
+            int rc = upload_float(dw, w, t.name, dt, t.elements());
+            if (rc) return rc;
+            continue;
+        }
+        MYNN_REQUIRE(it->second.dtype != MYNN_I8, MYNN_ERR_INVALID, "weights: %s is int8, a float tensor was expected", t.name.c_str());
+        std::vector<float> f;
+        to_f32(it->second, f);
+        void *d;
+        int rc = upload(dw, f.data(), f.size() * 4, &d);
+        if (rc) return rc;
+        dw.init.push_back(d);
+    }
+    return 0;
+}
+
 static mynn_device_weights *weights_upload_impl(const mynn_weights *w, const mynn_model_config *c) {
     if (!w || !c) {
         set_error("weights_upload: null argument");
         return nullptr;
+    }
+    if (c->arch) {
+        auto spec = arch_spec(c->arch);
+        if (!spec || spec->family != ModelSpec::LAYERED) {
+            set_error("weights_upload: no layered architecture %d", c->arch);
+            return nullptr;
+        }
+        auto dw = std::make_unique<mynn_device_weights>();
+        if (upload_arch(*dw, *w, *spec, c->dtype)) {
+            for (void *p : dw->owned) (void)hipFree(p);
+            return nullptr;
+        }
+        return dw.release();
     }
     auto e = w->entries.find("model.embed_tokens.weight");
     if (e == w->entries.end()) {
