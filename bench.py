@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Headline benchmark: batch-1 greedy decode of a TinyLlama-1.1B-shape int8 model on one MI355X.
 
-  python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload decode|prefill|attention|decode_batch|gemv]
+  python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload decode|prefill|attention|decode_batch|gemv|latent]
 
 `--workload prefill` times the matrix-core side of the same path instead: one step = one prefill
 pass of 8 prompts x 1024 tokens through the decoder executor (roofline bound: MFMA).
@@ -805,10 +805,145 @@ def decode_variants(mynn, cfg, weights, wset, prompt, K, tdt):
     return out
 
 
+# --workload latent: layers of the sizes real models have, the latent-attention design and the Llama graph at equal width,
+# feed-forward, heads and vocabulary (6 layer runs each; the design's are layer 0, two passes over 1..2, layer 3)
+LATENT_SIZES = {
+    "2048": dict(width=2048, heads=16, ff=5632, vocab=32000),
+    "3072": dict(width=3072, heads=24, ff=8192, vocab=64000),
+    "4096": dict(width=4096, heads=32, ff=14336, vocab=128256),
+}
+# launch of the design -> the like launch of the Llama graph
+LATENT_PAIRS = {
+    "decode": {"gemv_norm_latent_in": "gemv_norm_qkv", "latent_attention": "attention_rope_append|attention", "gemv_o": "gemv_o_residual",
+               "gemv_norm_gateup_geglu": "gemv_norm_gateup_swiglu", "gemv_down": "gemv_down_residual", "gemv_loop_in": "gemv_norm_qkv",
+               "latent_absorb_append": "rope_kv_append", "latent_merge_out": "gemv_o_residual", "gemv_norm_head": "gemv_norm_lm_head"},
+    "prefill": {"linear_latent_in": "linear_qkv", "linear_latent_kv": "linear_qkv", "latent_attention": "attention", "linear_o": "linear_o_residual",
+                "linear_gateup_geglu": "linear_gateup_swiglu", "linear_down": "linear_down_residual", "linear_loop_in": "linear_o_residual",
+                "residual_norm": "rms_norm", "residual_concat": "rms_norm", "latent_rotate_append": "rope_kv_append|rope_kv_append_k_v",
+                "latent_gather": "rope_kv_append|rope_kv_append_k_v"},
+}
+
+
+def latent_config(size):
+    H = size["heads"]
+    mix = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
+    layer = {"type": "latent_attention", "mixer": mix, "mlp": {"kind": "dense", "ff": size["ff"]}}
+    return {"architecture": "Dudilix", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-5}, "logit_scale": 1.0,
+            "embedding": {"bigram": {"buckets": 4096, "mul_prev": 127, "mul_cur": 31}}, "layers": [layer] * 4,
+            "loop": {"start": 1, "stop": 3, "times": 2}}
+
+
+def latent_main(args, mynn):
+    """Prefill of one prompt and batch-1 decode behind it, bf16, random weights: tokens/s of both models and, per launch,
+    the distance from the roofline beside the like launch of the Llama graph (int8 weights, bf16 activations)."""
+    import tempfile
+
+    import numpy as np
+    import torch
+
+    ctx, K, W = 2048, args.steps or 64, args.warmup or 16
+    max_seq, runs = 2560, 6
+    gen = torch.Generator(device="cuda")
+    gen.manual_seed(args.seed)
+    rng = np.random.default_rng(args.seed)
+
+    def per_kernel(profile, reps, kv_bytes):
+        agg = {}
+        for _ in range(reps):
+            for name, ms, nbytes, flops in profile():
+                a = agg.setdefault(name, [0, 0.0, 0.0, 0.0])
+                a[0] += 1
+                a[1] += ms
+                a[2] += nbytes + kv_bytes.get(name, 0.0)
+                a[3] += flops
+        out = {}
+        for name, (n, ms, nb, fl) in agg.items():
+            t = ms * 1e-3
+            if t <= 0:
+                continue
+            hbm, mfma = nb / t / 1e9 / HBM_PEAK_GBS, fl / t / 1e12 / MFMA_PEAK_TFLOPS
+            out[name] = {"us": round(t / n * 1e6, 2), "per_step": n // reps, "bound": "hbm" if hbm >= mfma else "mfma", "frac": round(max(hbm, mfma), 4)}
+        return out
+
+    def rate(fn, n, warm):
+        for _ in range(warm):
+            fn()
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for _ in range(n):
+            fn()
+        torch.cuda.synchronize()
+        return (time.perf_counter() - t0) / n
+
+    sizes = {}
+    for label, size in LATENT_SIZES.items():
+        ids = rng.integers(0, size["vocab"], ctx)
+        pos = np.arange(ctx)
+        res = {}
+        # ---- the design
+        with tempfile.TemporaryDirectory() as d:
+            with open(os.path.join(d, "config.json"), "w") as f:
+                json.dump(latent_config(size), f)
+            arch = mynn.Arch(d)
+        w = {}
+        for name, sh in arch.tensors():
+            w[name] = torch.ones(sh, dtype=torch.bfloat16, device="cuda") if len(sh) == 1 else \
+                (torch.randn(sh, generator=gen, device="cuda") * (1.0 if name in ("embed", "bigram") else sh[1] ** -0.5)).to(torch.bfloat16)
+        state = mynn.layered_state(arch, mynn.BF16, max_seq)
+        pre = mynn.LayeredDecoder(arch, w, mynn.BF16, max_seq, seq_q=ctx, state=state)
+        dec = mynn.LayeredDecoder(arch, w, mynn.BF16, max_seq, state=state)
+        t_pre = rate(lambda: pre.step_rows(ids, ctx, 0), 5, 2)
+        dec.decode_loop(1, ctx, W)
+        t_dec = rate(lambda: dec.decode_loop(1, ctx, K), 3, 1) / K
+        row = (512 + 64) * 2.0  # cached bytes of a token and layer run
+        res["latent"] = {"prefill_tok_s": round(ctx / t_pre), "decode_tok_s": round(1 / t_dec, 1), "launches_per_step": dec.stats()["launches_per_step"],
+                         "prefill": per_kernel(lambda: pre.profile(ids, pos, 0, ctx), 3, {}),
+                         "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, {"latent_attention": (ctx + 33) * row})}
+        pre.close(), dec.close()
+        del w, state
+        # ---- the Llama graph
+        H = size["heads"]
+        cfg = dict(n_layers=runs, hidden=size["width"], n_heads=H, n_kv_heads=H // 4, head_dim=128, ffn=size["ff"], vocab=size["vocab"],
+                   max_seq=max_seq, eps=1e-5, rope_theta=10000.0, dtype=mynn.BF16)
+        lw = make_weights(cfg, mynn.BF16, args.seed)
+        pre = mynn.Decoder(cfg, lw, seq_q=ctx)
+        dec = mynn.Decoder(cfg, lw, kv=pre.kv)
+        t_pre = rate(lambda: pre.step(ids, pos, 0, ctx), 5, 2)
+        dec.decode_loop(1, ctx, W)
+        t_dec = rate(lambda: dec.decode_loop(1, ctx, K), 3, 1) / K
+        kv = (ctx + 33) * 2.0 * cfg["n_kv_heads"] * 128 * 2
+        res["llama"] = {"prefill_tok_s": round(ctx / t_pre), "decode_tok_s": round(1 / t_dec, 1), "launches_per_step": dec.stats()["launches_per_step"],
+                        "prefill": per_kernel(lambda: pre.profile(ids, pos, 0, ctx), 3, {}),
+                        "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, {"attention_rope_append": kv, "attention": kv})}
+        pre.close(), dec.close()
+        del lw
+        torch.cuda.empty_cache()
+        # distance from the roofline relative to the like launch's: 1 / frac against 1 / frac
+        for phase, pairs in LATENT_PAIRS.items():
+            res["times_farther_" + phase] = {}
+            for mine, like in pairs.items():
+                other = next((o for o in like.split("|") if o in res["llama"][phase]), None)
+                if mine in res["latent"][phase] and other:
+                    a, b = res["latent"][phase][mine]["frac"], res["llama"][phase][other]["frac"]
+                    res["times_farther_" + phase][mine] = [other, round(b / max(a, 1e-6), 2)]
+        sizes[label] = res
+        print("bench.py: latent %s done" % label, file=sys.stderr, flush=True)
+    last = sizes["4096"]["latent"]
+    dom = max(last["decode"], key=lambda k: last["decode"][k]["us"] * last["decode"][k]["per_step"])
+    print(json.dumps({
+        "metric": "decode tok/s behind %d tokens, latent attention, width 4096, 6 layer runs" % ctx, "value": last["decode_tok_s"], "unit": "tok/s",
+        "n_gpus": 1, "steps": K, "warmup": W, "ms_per_step": round(1e3 / last["decode_tok_s"], 4), "higher_is_better": True, "scaling": "weak",
+        "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "latent attention (dim 128 + 64 rotated, value 128, latent 512) beside the Llama graph (int8 weights, head_dim 128, "
+                               "heads / 4 kv heads) at equal sizes; prompt of %d tokens, then decode" % ctx, "seed": args.seed, "sizes": sizes},
+        "roofline": {"bound": last["decode"][dom]["bound"], "kernel": dom, "frac": last["decode"][dom]["frac"], "peak": HBM_PEAK_GBS, "unit": "GB/s",
+                     "achieved": round(last["decode"][dom]["frac"] * HBM_PEAK_GBS, 1), "avg_launch_us": last["decode"][dom]["us"]}}))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
-    ap.add_argument("--workload", choices=["decode", "prefill", "attention", "decode_batch", "gemv"], default="decode")
+    ap.add_argument("--workload", choices=["decode", "prefill", "attention", "decode_batch", "gemv", "latent"], default="decode")
     ap.add_argument("--steps", type=int, default=None, help="default 256 (decode) / 5 (prefill)")
     ap.add_argument("--warmup", type=int, default=None, help="default 16 (decode) / 2 (prefill)")
     ap.add_argument("--dtype", choices=["f16", "bf16"], default="f16")
@@ -872,6 +1007,8 @@ def main():
         return decode_batch_main(args, mynn)
     if args.workload == "gemv":
         return gemv_main(args, mynn)
+    if args.workload == "latent":
+        return latent_main(args, mynn)
     K = 256 if args.steps is None else args.steps
     W = 16 if args.warmup is None else args.warmup
     # the cache of configs[2] holds 128 + 256 rows; longer runs get a longer cache (whole 128-row pages, up to the 2048 rows

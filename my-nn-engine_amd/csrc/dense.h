@@ -62,8 +62,16 @@ int residual_norm_rows(void *act, const ResidualNorm &r, int pro, int first, int
 // PRO_ROWS: act = T [K]; else r describes the row (K = ld or 2 ld).
 enum { DENSE_T = 0, DENSE_F32 = 1, DENSE_GEGLU = 2 };
 bool dense_gemv_supported(int K);
+// cand (DENSE_F32): every workgroup leaves its largest output there, *n_cand of them (at most kGreedyCands); greedy_pick
+// takes the best, the last maximum as argmax_rows does, and moves the loop state on.
+struct GreedyCand {
+    float value;
+    int index;  // -1: none
+};
+constexpr int kGreedyCands = 1024;
 int dense_gemv(void *out, const void *act, const ResidualNorm *r, int pro, const void *w, int N, int K, int store, const float *scale,
-               int dtype, hipStream_t s);
+               int dtype, hipStream_t s, GreedyCand *cand = nullptr, int *n_cand = nullptr);
+int greedy_pick(int32_t *out, const GreedyCand *cand, int n, AdvanceState adv, hipStream_t s);
 
 // any number of rows: act [M, K]; 16-bit types on the matrix cores' 16-bit product, f32 on their f32 product
 int dense_gemm(void *out, const void *act, const void *w, int M, int N, int K, int store, const float *scale, int dtype, hipStream_t s);

@@ -212,11 +212,26 @@ int residual_norm_rows(void *act, const ResidualNorm &r, int pro, int first, int
     });
 }
 
+// best (value, index) of a workgroup's threads, in thread 0
+__device__ inline void workgroup_best(float &bv, int &bi, GreedyCand *best) {
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) {
+        const float ov = __shfl_xor(bv, off, kWave);
+        const int oi = __shfl_xor(bi, off, kWave);
+        if (oi >= 0) argmax_take(bv, bi, ov, oi);
+    }
+    if ((threadIdx.x & 63) == 0) best[threadIdx.x >> 6] = GreedyCand{bv, bi};
+    __syncthreads();
+    if (threadIdx.x == 0)
+        for (int w = 1; w < kRowWaves; w++)
+            if (best[w].index >= 0) argmax_take(bv, bi, best[w].value, best[w].index);
+}
+
 // ---- one-row linear -----------------------------------------------------------------------------------------------------
 // A wave's row group: R rows; GEGLU: R / 2 gate rows and the R / 2 up rows 32 further on.
 template <typename T, int R, int PRO, int STORE>
 __global__ __launch_bounds__(kRowThreads) void dense_gemv_kernel(const T *w, const void *act_in, int N, int K, int groups, int total_waves,
-                                                                 void *out, const float *scale, ResidualNorm r) {
+                                                                 void *out, const float *scale, ResidualNorm r, GreedyCand *cand) {
     constexpr int E = 16 / (int)sizeof(T);  // weights per 16-byte load
     constexpr int UN = sizeof(T) == 2 ? 4 : 4;
     extern __shared__ __align__(16) float act[];  // [K]
@@ -273,6 +288,8 @@ __global__ __launch_bounds__(kRowThreads) void dense_gemv_kernel(const T *w, con
     }
     __syncthreads();
 
+    float bv = -INFINITY;  // this lane's best output so far (cand)
+    int bi = -1;
     bool first = true;
     for (; g < groups; g += total_waves) {
         float acc[R];
@@ -314,17 +331,61 @@ __global__ __launch_bounds__(kRowThreads) void dense_gemv_kernel(const T *w, con
                 if (lane == i) mine = acc[i];
             const int n = g * R + lane;
             if (lane < R && n < N) {
-                if constexpr (STORE == DENSE_F32) ((float *)out)[n] = scale ? mine * *scale : mine;
-                else Elem<T>::st((T *)out, n, mine);
+                if constexpr (STORE == DENSE_F32) {
+                    const float v = scale ? mine * *scale : mine;
+                    ((float *)out)[n] = v;
+                    argmax_take(bv, bi, v, n);
+                } else Elem<T>::st((T *)out, n, mine);
             }
         }
     }
+    if constexpr (STORE == DENSE_F32) {
+        if (cand) {
+            __shared__ GreedyCand best[kRowWaves];
+            workgroup_best(bv, bi, best);
+            if (threadIdx.x == 0) cand[blockIdx.x] = GreedyCand{bv, bi};
+        }
+    }
+}
+
+// the best of the workgroups' candidates (the last maximum wins), as argmax_rows leaves it
+__global__ __launch_bounds__(256) void greedy_pick_kernel(int32_t *out, const GreedyCand *cand, int n, AdvanceState adv) {
+    __shared__ GreedyCand best[4];
+    int st_step = 0, st_past = 0, st_active = 0;
+    int64_t st_pos = 0;
+    if (adv.ids && threadIdx.x == 0) {
+        st_step = *adv.step;
+        st_pos = adv.pos[0];
+        st_past = *adv.past;
+        st_active = *adv.active;
+    }
+    float bv = -INFINITY;
+    int bi = -1;
+    for (int i = threadIdx.x; i < n; i += 256)
+        if (cand[i].index >= 0) argmax_take(bv, bi, cand[i].value, cand[i].index);
+    workgroup_best(bv, bi, best);
+    if (threadIdx.x) return;
+    out[0] = bi;
+    if (adv.ids) {
+        if (st_step < adv.cap) adv.tokens[st_step] = bi;
+        *adv.step = st_step + 1;
+        adv.ids[0] = bi;
+        adv.pos[0] = st_pos + 1;
+        *adv.past = st_past + 1;
+        *adv.active = st_active + 1;
+    }
+}
+int greedy_pick(int32_t *out, const GreedyCand *cand, int n, AdvanceState adv, hipStream_t s) {
+    MYNN_REQUIRE(out && cand && n > 0, MYNN_ERR_INVALID, "greedy pick: bad operand");
+    MYNN_LAUNCH(greedy_pick_kernel, dim3(1), dim3(256), 0, s, out, cand, n, adv);
+    return launch_status("greedy_pick_kernel");
 }
 
 bool dense_gemv_supported(int K) { return K % 64 == 0 && (size_t)K * 4 <= kRowLdsMax; }
 
 template <typename T, int R, int PRO, int STORE>
-static int launch_gemv(void *out, const void *act, const ResidualNorm &r, const void *w, int N, int K, const float *scale, hipStream_t s) {
+static int launch_gemv(void *out, const void *act, const ResidualNorm &r, const void *w, int N, int K, const float *scale, hipStream_t s,
+                       GreedyCand *cand, int *n_cand) {
     const int groups = STORE == DENSE_GEGLU ? (N / 2 + R / 2 - 1) / (R / 2) : (N + R - 1) / R;
     const size_t lds = (size_t)K * 4;
     const int per_cu = (int)(kRowLdsMax / lds) < 4 ? (int)(kRowLdsMax / lds) : 4;
@@ -333,12 +394,14 @@ static int launch_gemv(void *out, const void *act, const ResidualNorm &r, const 
     const int blocks = ((groups + passes - 1) / passes + kRowWaves - 1) / kRowWaves;
     auto kernel = dense_gemv_kernel<T, R, PRO, STORE>;
     if (lds > 60 * 1024) { int rc = allow_lds(kernel); if (rc) return rc; }
-    MYNN_LAUNCH(kernel, dim3(blocks), dim3(kRowThreads), lds, s, (const T *)w, act, N, K, groups, blocks * kRowWaves, out, scale, r);
+    MYNN_LAUNCH(kernel, dim3(blocks), dim3(kRowThreads), lds, s, (const T *)w, act, N, K, groups, blocks * kRowWaves, out, scale, r, cand);
+    if (n_cand) *n_cand = blocks;
     return launch_status("dense_gemv_kernel");
 }
 
 int dense_gemv(void *out, const void *act, const ResidualNorm *r, int pro, const void *w, int N, int K, int store, const float *scale,
-               int dtype, hipStream_t s) {
+               int dtype, hipStream_t s, GreedyCand *cand, int *n_cand) {
+    MYNN_REQUIRE(!cand || store == DENSE_F32, MYNN_ERR_INVALID, "dense gemv: candidates of store %d", store);
     MYNN_REQUIRE(out && w && N > 0 && dense_gemv_supported(K), MYNN_ERR_INVALID, "dense gemv: N=%d K=%d", N, K);
     MYNN_REQUIRE(store != DENSE_GEGLU || N % 64 == 0, MYNN_ERR_INVALID, "dense gemv: %d interleaved gate/up rows", N);
     if (pro == PRO_ROWS) MYNN_REQUIRE(act, MYNN_ERR_INVALID, "dense gemv: null activation");
@@ -353,15 +416,15 @@ int dense_gemv(void *out, const void *act, const ResidualNorm *r, int pro, const
         using T = std::remove_pointer_t<decltype(t)>;
         if (pro == PRO_RESIDUAL_CONCAT) {
             MYNN_REQUIRE(store == DENSE_F32, MYNN_ERR_UNSUPPORTED, "dense gemv: concatenated row with store %d", store);
-            return launch_gemv<T, 2, PRO_RESIDUAL_CONCAT, DENSE_F32>(out, act, rr, w, N, K, scale, s);
+            return launch_gemv<T, 2, PRO_RESIDUAL_CONCAT, DENSE_F32>(out, act, rr, w, N, K, scale, s, cand, n_cand);
         }
         if (pro == PRO_RESIDUAL_NORM) {
-            if (store == DENSE_GEGLU) return launch_gemv<T, 4, PRO_RESIDUAL_NORM, DENSE_GEGLU>(out, act, rr, w, N, K, scale, s);
-            if (store == DENSE_F32) return launch_gemv<T, 4, PRO_RESIDUAL_NORM, DENSE_F32>(out, act, rr, w, N, K, scale, s);
-            return launch_gemv<T, 2, PRO_RESIDUAL_NORM, DENSE_T>(out, act, rr, w, N, K, scale, s);
+            if (store == DENSE_GEGLU) return launch_gemv<T, 4, PRO_RESIDUAL_NORM, DENSE_GEGLU>(out, act, rr, w, N, K, scale, s, cand, n_cand);
+            if (store == DENSE_F32) return launch_gemv<T, 4, PRO_RESIDUAL_NORM, DENSE_F32>(out, act, rr, w, N, K, scale, s, cand, n_cand);
+            return launch_gemv<T, 2, PRO_RESIDUAL_NORM, DENSE_T>(out, act, rr, w, N, K, scale, s, cand, n_cand);
         }
         MYNN_REQUIRE(store == DENSE_T, MYNN_ERR_UNSUPPORTED, "dense gemv: plain row with store %d", store);
-        return launch_gemv<T, 2, PRO_ROWS, DENSE_T>(out, act, rr, w, N, K, scale, s);
+        return launch_gemv<T, 2, PRO_ROWS, DENSE_T>(out, act, rr, w, N, K, scale, s, cand, n_cand);
     });
 }
 

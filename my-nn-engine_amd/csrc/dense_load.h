@@ -32,6 +32,18 @@ template <> __device__ inline void load8<float>(const float *p, float *f) {
     *(float4 *)(f + 4) = *(const float4 *)(p + 4);
 }
 
+// eight values of T, kept as loaded until they are used
+template <typename T> struct Row8 {
+    U4 v;
+    __device__ void get(const T *p) { v = *(const U4 *)p; }
+    __device__ void widen(float *f) const { widen8<T>(v, f); }
+};
+template <> struct Row8<float> {
+    float4 a, b;
+    __device__ void get(const float *p) { a = *(const float4 *)p; b = *(const float4 *)(p + 4); }
+    __device__ void widen(float *f) const { *(float4 *)f = a; *(float4 *)(f + 4) = b; }
+};
+
 __device__ inline float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
 // 0.5 z (1 + tanh(u)) = z * sigmoid(2 u), u = sqrt(2 / pi) (z + 0.044715 z^3)
 __device__ inline float gelu_tanh_arg(float z) { return 1.5957691216057308f * fmaf(0.044715f * z * z, z, z); }

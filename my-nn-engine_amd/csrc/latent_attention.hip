@@ -9,6 +9,7 @@
 //   expanded (prompts): K = W_uk c, V = W_uv c for every visible token by one GEMM, then flash attention over query / key
 //     width dim + rot_dim and value width vdim (latent_prefill_kernel), the gate in the store.
 // latent_absorbed_plain_kernel is the absorbed product for f32 and for shapes the matrix-core kernel has no form for.
+#include <algorithm>
 #include <type_traits>
 
 #include "dense_load.h"
@@ -36,7 +37,7 @@ __device__ inline void rotate_pair(const LatentParams &p, int pos, int i, float 
 }
 
 // ---- prepare: workgroup x == 0 of a row makes the cache row, the others the queries ---------------------------------
-constexpr int kPrepThreads = 256, kPrepCols = 512;
+constexpr int kPrepThreads = 256, kPrepCols = 128;
 template <typename T, bool ABSORB>
 __global__ __launch_bounds__(kPrepThreads) void latent_prepare_kernel(LatentParams p) {
     __shared__ float sm[kPrepThreads * 8 + 8];
@@ -46,6 +47,8 @@ __global__ __launch_bounds__(kPrepThreads) void latent_prepare_kernel(LatentPara
     if (blockIdx.x == 0) {
         const T *lat = proj + d.qcols(), *kr = lat + d.rp;
         T *dst = (T *)p.cache + latent_row(p, b, pos) * d.lw();
+        // (one sequence, expanded form: the row also goes where the expansion reads it)
+        T *c2 = !ABSORB && p.B == 1 ? (T *)p.c_rows + (size_t)pos * d.rp : nullptr, *r2 = c2 ? (T *)p.rot_rows + (size_t)pos * d.rotp : nullptr;
         float ss = 0.f;
         for (int k = tid; k < d.rank; k += kPrepThreads) {
             const float v = Elem<T>::ld(lat, k);
@@ -55,13 +58,20 @@ __global__ __launch_bounds__(kPrepThreads) void latent_prepare_kernel(LatentPara
         if ((tid & 63) == 0) sm[tid >> 6] = ss;
         __syncthreads();
         const float inv = 1.0f / sqrtf((sm[0] + sm[1] + sm[2] + sm[3]) / (float)d.rank + p.eps);
-        for (int k = tid; k < d.rp; k += kPrepThreads)
-            Elem<T>::st(dst, k, k < d.rank ? Elem<T>::ld(lat, k) * inv * Elem<T>::ld((const T *)p.norm_w, k) : 0.f);
+        for (int k = tid; k < d.rp; k += kPrepThreads) {
+            const float v = k < d.rank ? Elem<T>::ld(lat, k) * inv * Elem<T>::ld((const T *)p.norm_w, k) : 0.f;
+            Elem<T>::st(dst, k, v);
+            if (c2) Elem<T>::st(c2, k, v);
+        }
         for (int i = tid; i < d.rotp / 2; i += kPrepThreads) {
             float u = Elem<T>::ld(kr, 2 * i), v = Elem<T>::ld(kr, 2 * i + 1);
             rotate_pair(p, pos, i, u, v);
             Elem<T>::st(dst, d.rp + 2 * i, u);
             Elem<T>::st(dst, d.rp + 2 * i + 1, v);
+            if (r2) {
+                Elem<T>::st(r2, 2 * i, u);
+                Elem<T>::st(r2, 2 * i + 1, v);
+            }
         }
         return;
     }
@@ -114,7 +124,7 @@ __global__ __launch_bounds__(kPrepThreads) void latent_prepare_kernel(LatentPara
 }
 
 int latent_prepare(const LatentParams &p, bool absorb, int dtype, hipStream_t s) {
-    MYNN_REQUIRE(p.proj && p.norm_w && p.cache && p.rot && p.d_past && (!absorb || (p.ukv && p.q_abs)), MYNN_ERR_INVALID, "latent prepare: null operand");
+    MYNN_REQUIRE(p.proj && p.norm_w && p.cache && p.rot && p.d_past && (!absorb || (p.ukv && p.q_abs)) && (absorb || p.B > 1 || (p.c_rows && p.rot_rows)), MYNN_ERR_INVALID, "latent prepare: null operand");
     MYNN_REQUIRE((long)p.B * p.S <= 65535, MYNN_ERR_UNSUPPORTED, "latent prepare: %d rows", p.B * p.S);
     const int nchunk = (p.d.rp + kPrepCols - 1) / kPrepCols;
     const dim3 grid(absorb ? 1 + p.d.H * nchunk : 2, p.B * p.S);
@@ -139,9 +149,9 @@ __device__ __host__ inline int latent_range(int active, int nsplit) {
 // or by halves of the row for MT == 1), every wave then takes the softmax of all rows and adds its own 32-column blocks
 // of P . C.  CB: 32-column blocks per wave.
 template <typename T, int MT, int CB>
-__global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p) {
+__global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, unsigned div) {
     constexpr int KS = MT == 1 ? 2 : 1;  // partial score products per (key, query)
-    constexpr int NL = 2 * CB + 2;       // 16-byte pieces of a tile per thread
+    constexpr int NL = 2 * CB + 2, NQ = MT * (CB + 1);  // 16-byte pieces of a tile / of the queries per thread
     constexpr int SST = kTile + 4;
     extern __shared__ __align__(16) char smem[];
     const LatentDims &d = p.d;
@@ -155,13 +165,6 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p) {
     const int last_q = min(r0 + 16 * MT - 1, nrows - 1) / d.H;       // the furthest query of the workgroup
     const int k0 = split * range, k1 = min(min(past + p.S, k0 + range), past + last_q + 1);
 
-    // queries to LDS (rows past the end: zeros)
-    for (int i = tid; i < 16 * MT * cpr; i += 256) {
-        const int r = i / cpr, c = i % cpr;
-        U4 v = U4{0u, 0u, 0u, 0u};
-        if (r0 + r < nrows) v = *(const U4 *)((const T *)p.q_abs + ((size_t)b * nrows + r0 + r) * lw + c * 8);
-        *(U4 *)(Qs + r * ldc + c * 8) = v;
-    }
     int bound[MT];  // keys the row of this lane's column sees
 #pragma unroll
     for (int m = 0; m < MT; m++) bound[m] = past + min(r0 + 16 * m + col, nrows - 1) / d.H + 1;
@@ -183,28 +186,42 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p) {
     // is asked for one tile ahead of the loads that need it)
     auto page_of = [&](int t) { return table ? table[(k0 + min(t, ntiles - 1) * kTile) >> psh] : 0; };
     U4 pre[NL];
+    // idx / cpr for idx < 8192, cpr <= 128 by a multiplication: div = ceil(2^20 / cpr), so idx * (div * cpr - 2^20) < 2^20
+    auto row_of = [&](int idx) { return (int)(((unsigned)idx * div) >> 20); };
     auto load_tile = [&](int t, int page) {
         const int t0 = k0 + t * kTile;
 #pragma unroll
         for (int i = 0; i < NL; i++) {
-            const int idx = min(tid + i * 256, kTile * cpr - 1);
-            const int key = min(t0 + idx / cpr, k1 - 1);
+            const int idx = min(tid + i * 256, kTile * cpr - 1), r = row_of(idx);
+            const int key = min(t0 + r, k1 - 1);
             const size_t row = table ? ((size_t)page << psh) + (key & pmask) : (size_t)b * p.max_seq + key;
-            pre[i] = *(const U4 *)((const T *)p.cache + row * lw + (idx % cpr) * 8);
+            pre[i] = *(const U4 *)((const T *)p.cache + row * lw + (idx - r * cpr) * 8);
         }
     };
     int page_next = 0;
     if (ntiles) {
         load_tile(0, page_of(0));
         page_next = page_of(1);
+        // queries to LDS (rows past the end: zeros), all of a thread's pieces requested together
+        U4 qv[NQ];
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            const int idx = min(tid + i * 256, 16 * MT * cpr - 1), r = row_of(idx);
+            qv[i] = *(const U4 *)((const T *)p.q_abs + ((size_t)b * nrows + min(r0 + r, nrows - 1)) * lw + (idx - r * cpr) * 8);
+        }
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            const int idx = tid + i * 256, r = row_of(idx);
+            if (idx < 16 * MT * cpr) *(U4 *)(Qs + r * ldc + (idx - r * cpr) * 8) = r0 + r < nrows ? qv[i] : U4{0u, 0u, 0u, 0u};
+        }
     }
     const int nks = lw >> 5, nblk = d.rp >> 5;
     for (int t = 0; t < ntiles; t++) {
         __syncthreads();  // the tile before is no longer read
 #pragma unroll
         for (int i = 0; i < NL; i++) {
-            const int idx = tid + i * 256;
-            if (idx < kTile * cpr) *(U4 *)(Cs + (idx / cpr) * ldc + (idx % cpr) * 8) = pre[i];
+            const int idx = tid + i * 256, r = row_of(idx);
+            if (idx < kTile * cpr) *(U4 *)(Cs + r * ldc + (idx - r * cpr) * 8) = pre[i];
         }
         __syncthreads();
         if (t + 1 < ntiles) {
@@ -215,9 +232,24 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p) {
         {
             const int kt = wave & 1, other = wave >> 1;
             const int qt = MT == 1 ? 0 : other;
-            lf4_t s4 = {0.f, 0.f, 0.f, 0.f};
+            lf4_t s4 = {0.f, 0.f, 0.f, 0.f}, s5 = {0.f, 0.f, 0.f, 0.f};
             const T *ca = Cs + (kt * 16 + col) * ldc + quad * 8, *qb = Qs + (qt * 16 + col) * ldc + quad * 8;
-            for (int ks = MT == 1 ? other : 0; ks < nks; ks += KS) s4 = MfmaL16<T>::run(*(const U4 *)(ca + ks * 32), *(const U4 *)(qb + ks * 32), s4);
+            // (four steps at a time: their reads are in flight together; steps past the row multiply zeros)
+            for (int k4 = MT == 1 ? other : 0; k4 < nks; k4 += 4 * KS) {
+                U4 fa[4], fb[4];
+#pragma unroll
+                for (int j = 0; j < 4; j++) {
+                    const int ks = k4 + j * KS, kc = min(ks, nks - 1);
+                    fa[j] = *(const U4 *)(ca + kc * 32);
+                    fb[j] = *(const U4 *)(qb + kc * 32);
+                    if (ks >= nks) fb[j] = U4{0u, 0u, 0u, 0u};
+                }
+                s4 = MfmaL16<T>::run(fa[0], fb[0], s4);
+                s5 = MfmaL16<T>::run(fa[1], fb[1], s5);
+                s4 = MfmaL16<T>::run(fa[2], fb[2], s4);
+                s5 = MfmaL16<T>::run(fa[3], fb[3], s5);
+            }
+            s4 += s5;
             float *dst = Ss + ((MT == 1 ? other : 0) * 16 * MT + qt * 16 + col) * SST + kt * 16 + quad * 4;
             *(float4 *)dst = float4{s4[0], s4[1], s4[2], s4[3]};
         }
@@ -378,9 +410,12 @@ __global__ __launch_bounds__(256) void latent_absorbed_plain_kernel(LatentParams
 
 static bool absorbed_mfma_supported(const LatentDims &d, int dtype) { return dtype == MYNN_BF16 && d.rp <= 512 && d.rotp <= 128; }
 
+// 16-row tiles per workgroup: one while there are few rows (more workgroups, each with less to do), else two per key read
+static int absorbed_row_tiles(int B, int S, const LatentDims &d) { return S * d.H <= 16 || (long)B * S * d.H <= 64 ? 1 : 2; }
+
 int latent_absorbed_splits(int B, int S, const LatentDims &d, int max_seq, int dtype) {
     if (!absorbed_mfma_supported(d, dtype)) return 1;
-    const int mt = S * d.H <= 16 ? 1 : 2;
+    const int mt = absorbed_row_tiles(B, S, d);
     const long tiles = (long)B * ((S * d.H + 16 * mt - 1) / (16 * mt));
     long n = 512 / tiles;
     const long most = (max_seq + kMinRange - 1) / kMinRange;
@@ -403,13 +438,14 @@ int latent_attention_absorbed(const LatentParams &p, int dtype, hipStream_t s) {
             return launch_status("latent_absorbed_plain_kernel");
         });
     }
-    const int mt = p.S * d.H <= 16 ? 1 : 2;
+    const int mt = absorbed_row_tiles(p.B, p.S, d);
+    const unsigned cpr = d.lw() >> 3;
     const dim3 grid(p.nsplit, (p.S * d.H + 16 * mt - 1) / (16 * mt), p.B);
     MYNN_REQUIRE(grid.y <= 65535 && grid.z <= 65535, MYNN_ERR_UNSUPPORTED, "latent attention: %d rows of %d heads", p.S, d.H);
     const size_t lds = (size_t)(kTile + 16 * mt) * (d.lw() + 8) * 2 + (size_t)(mt == 1 ? 2 : 1) * 16 * mt * (kTile + 4) * 4;
     auto go = [&](auto kernel) {
         if (lds > 60 * 1024) MYNN_HIP(hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-        MYNN_LAUNCH(kernel, grid, dim3(256), lds, s, p);
+        MYNN_LAUNCH(kernel, grid, dim3(256), lds, s, p, ((1u << 20) + cpr - 1) / cpr);
         return launch_status("latent_absorbed_kernel");
     };
     const int nblk = d.rp >> 5;
@@ -422,13 +458,21 @@ constexpr int kMaxRanges = 128;
 template <typename T>
 __global__ __launch_bounds__(256) void latent_out_kernel(LatentParams p) {
     extern __shared__ __align__(16) char smem[];
-    float *o = (float *)smem;  // [rp]
+    float *o = (float *)smem;  // [rp], then the partial sums
     __shared__ float wgt[kMaxRanges];
     const LatentDims &d = p.d;
     const int h = blockIdx.y, row = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const size_t at = ((size_t)row * d.H + h) * p.nsplit;
     // ranges that hold a key this row sees
     const int live = p.nsplit == 1 ? 1 : (*p.d_past + row % p.S) / latent_range(*p.d_past + p.S, p.nsplit) + 1;
+    // this wave's eight rows of W_uv (a latent of up to 512 values: one piece per lane) are on their way first
+    const int v0 = blockIdx.x * 32 + wave * 8;
+    const T *uv = (const T *)p.ukv + ((size_t)d.H * d.dimp + (size_t)h * d.vdimp + v0) * d.rp;
+    const bool have = lane * 8 < d.rp;
+    Row8<T> wr[8];
+#pragma unroll
+    for (int j = 0; j < 8; j++)
+        if (have) wr[j].get(uv + (size_t)j * d.rp + lane * 8);
     if (wave == 0) {
         float m = -INFINITY;
         for (int i = lane; i < live; i += 64) m = fmaxf(m, p.part_ml[(at + i) * 2]);
@@ -439,23 +483,36 @@ __global__ __launch_bounds__(256) void latent_out_kernel(LatentParams p) {
         for (int i = lane; i < live; i += 64) wgt[i] = expf(p.part_ml[(at + i) * 2] - m) / l;
     }
     __syncthreads();
+    // thread = (four latents, every ng-th range), the groups' sums meet in LDS; eight ranges in flight per thread
+    const int n4 = d.rp >> 2, ng = 256 / min(n4, 256), grp = tid / n4;
+    float *acc_s = o + d.rp;  // [ng][rp]
+    for (int c4 = tid - grp * n4; c4 < n4 && grp < ng; c4 += 256) {
+        float4 a = float4{0.f, 0.f, 0.f, 0.f};
+        const float *src = p.part_o + at * d.rp + c4 * 4;
+#pragma unroll 8
+        for (int i = grp; i < live; i += ng) {
+            const float4 v = *(const float4 *)(src + (size_t)i * d.rp);
+            const float w = wgt[i];
+            a.x = fmaf(w, v.x, a.x); a.y = fmaf(w, v.y, a.y); a.z = fmaf(w, v.z, a.z); a.w = fmaf(w, v.w, a.w);
+        }
+        *(float4 *)(acc_s + grp * d.rp + c4 * 4) = a;
+    }
+    __syncthreads();
     for (int k = tid; k < d.rp; k += 256) {
         float a = 0.f;
-        for (int i = 0; i < live; i++) a = fmaf(wgt[i], p.part_o[(at + i) * d.rp + k], a);
+        for (int i = 0; i < ng; i++) a += acc_s[i * d.rp + k];
         o[k] = a;
     }
     __syncthreads();
     const float g = sigmoidf(Elem<T>::ld((const T *)p.proj, (size_t)row * d.n_in() + d.qcols() + d.lw() + h));
-    // eight value rows per wave
-    const int v0 = blockIdx.x * 32 + wave * 8;
     float acc[8];
 #pragma unroll
     for (int j = 0; j < 8; j++) {
         acc[j] = 0.f;
-        const T *w = (const T *)p.ukv + ((size_t)d.H * d.dimp + (size_t)h * d.vdimp + v0 + j) * d.rp;
         for (int c = lane * 8; c < d.rp; c += 512) {
             float f[8];
-            load8<T>(w + c, f);
+            if (c < 512) wr[j].widen(f);
+            else load8<T>(uv + (size_t)j * d.rp + c, f);
 #pragma unroll
             for (int e = 0; e < 8; e++) acc[j] = fmaf(f[e], o[c + e], acc[j]);
         }
@@ -473,7 +530,10 @@ int latent_merge_out(const LatentParams &p, int dtype, hipStream_t s) {
     const dim3 grid(p.d.vdimp / 32, p.d.H, p.B * p.S);
     return dispatch_dense(dtype, [&](auto *t) {
         using T = std::remove_pointer_t<decltype(t)>;
-        MYNN_LAUNCH(latent_out_kernel<T>, grid, dim3(256), (size_t)p.d.rp * 4, s, p);
+        const int ng = 256 / std::min(p.d.rp >> 2, 256);
+        const size_t lds = (size_t)(1 + ng) * p.d.rp * 4;
+        MYNN_REQUIRE(lds <= 60 * 1024, MYNN_ERR_UNSUPPORTED, "latent merge: latent of %d values", p.d.rank);
+        MYNN_LAUNCH(latent_out_kernel<T>, grid, dim3(256), lds, s, p);
         return launch_status("latent_out_kernel");
     });
 }

@@ -57,6 +57,7 @@ struct LayeredNet {
     void *act = nullptr, *proj = nullptr, *attn = nullptr, *y = nullptr, *hmid = nullptr, *q_abs = nullptr;
     void *c_rows = nullptr, *rot_rows = nullptr, *kv = nullptr;
     float *part_o = nullptr, *part_ml = nullptr;
+    GreedyCand *cand = nullptr;
     bool gemv = false;            // every linear fits the one-row kernel
 };
 void destroy_layered(Model &m) {
@@ -227,7 +228,7 @@ int build_layered(Model &m, void **state) {
     const size_t o_c = plan.take(c_rows * eb), o_r = plan.take(rot_rows * eb), o_kv = plan.take(kv * eb);
     const size_t o_l = plan.take((size_t)rows * s.vocab * 4), o_sc = plan.take(32 + (size_t)c.batch * 4);
     const size_t o_ids = plan.take((size_t)rows * 8), o_pos = plan.take((size_t)c.seq_q * 8), o_tok = plan.take((size_t)m.token_cap * 4);
-    const size_t o_ls = plan.take(4);
+    const size_t o_ls = plan.take(4), o_cand = plan.take(kGreedyCands * sizeof(GreedyCand));
     m.arena_bytes = plan.off;
     MYNN_HIP(hipMalloc((void **)&m.arena, m.arena_bytes));
     MYNN_HIP(hipMemset(m.arena, 0, m.arena_bytes));
@@ -239,6 +240,7 @@ int build_layered(Model &m, void **state) {
     m.d_past = (int32_t *)(m.arena + o_sc); m.d_active = m.d_past + 1; m.d_step = m.d_past + 2; m.d_next = m.d_past + 8;
     m.d_ids = (int64_t *)(m.arena + o_ids); m.d_pos = (int64_t *)(m.arena + o_pos); m.d_tokens = (int32_t *)(m.arena + o_tok);
     n.logit_scale = (float *)(m.arena + o_ls);
+    n.cand = (GreedyCand *)(m.arena + o_cand);
     MYNN_HIP(hipMemcpy(n.logit_scale, &s.logit_scale, 4, hipMemcpyHostToDevice));
     m.next_stage = align_up((size_t)c.batch * 4, 256);
     m.stage_bytes = align_up((size_t)rows * 8 + (size_t)c.seq_q * 8 + 64 + (size_t)m.token_cap * 4, 256) + 256 + m.next_stage;
@@ -319,8 +321,12 @@ int latent_attention(Stream &st, int run, const LayerWeights &w, const MixerSpec
     } else {
         const int L = m.h_past + S;
         for (int b = 0; b < B; b++) {
-            note(m, "latent_gather", 2.0 * L * d.lw() * eb);
-            TRY(latent_gather(p, b, L, c.dtype, m.stream));
+            // (one sequence: latent_prepare has put the new tokens' rows in place already)
+            const int gather = B == 1 ? m.h_past : L;
+            if (gather) {
+                note(m, "latent_gather", 2.0 * gather * d.lw() * eb);
+                TRY(latent_gather(p, b, gather, c.dtype, m.stream));
+            }
             note(m, "linear_latent_kv", ((double)L * d.rp + (double)w.ukv.N * w.ukv.K + (double)L * w.ukv.N) * eb, 2.0 * L * w.ukv.N * w.ukv.K);
             TRY(dense_gemm(n.kv, n.c_rows, w.ukv.w, L, w.ukv.N, w.ukv.K, DENSE_T, nullptr, c.dtype, m.stream));
             note(m, "latent_attention", (double)(S * (d.qcols() + d.acols()) + L * (d.kvcols() + d.rotp)) * eb,
@@ -377,23 +383,27 @@ int enqueue_layered(Model &m) {
 
     // logits of the rows the caller asked for
     const int cnt = m.sel_count, V = s.vocab;
+    AdvanceState adv{};  // a batch-1 decode model's step also moves the loop state on
+    if (c.batch * c.seq_q == 1) adv = AdvanceState{m.d_ids, m.d_pos, m.d_past, m.d_active, m.d_tokens, m.d_step, m.token_cap};
     if (cnt) {
         ResidualNorm row = st.row(n.w->final_norm);
         row.x_out = nullptr;
         if (st.one) {
+            int n_cand = 0;
             note(m, "gemv_norm_head", (double)V * n.ld * eb + st.row_bytes(eb) + V * 4.0, 2.0 * V * n.ld);
-            TRY(dense_gemv(m.logits, nullptr, &row, PRO_RESIDUAL_NORM, n.w->head.w, V, n.ld, DENSE_F32, n.logit_scale, dt, m.stream));
+            TRY(dense_gemv(m.logits, nullptr, &row, PRO_RESIDUAL_NORM, n.w->head.w, V, n.ld, DENSE_F32, n.logit_scale, dt, m.stream, n.cand, &n_cand));
+            note(m, adv.ids ? "greedy_advance" : "greedy_pick", n_cand * 8.0);
+            TRY(greedy_pick(m.d_next, n.cand, n_cand, adv, m.stream));
         } else {
             note(m, "residual_norm", cnt * (st.row_bytes(eb) + n.ld * eb));
             TRY(residual_norm_rows(n.act, row, PRO_RESIDUAL_NORM, m.sel_first, m.sel_stride, cnt, dt, m.stream));
             note(m, "linear_head", (double)(V + cnt) * n.ld * eb + (double)cnt * V * 4, 2.0 * cnt * V * n.ld);
             TRY(dense_gemm(m.logits, n.act, n.w->head.w, cnt, V, n.ld, DENSE_F32, n.logit_scale, dt, m.stream));
         }
-        // greedy token of every sequence whose last row is among them; a batch-1 decode step also moves the loop state on
+        // greedy token of every sequence whose last row is among them
         const float *lg = (const float *)m.logits;
-        if (S == 1 || (cnt == c.batch && (c.batch > 1 || m.sel_first == S - 1))) {
-            AdvanceState adv{};
-            if (c.batch * c.seq_q == 1) adv = AdvanceState{m.d_ids, m.d_pos, m.d_past, m.d_active, m.d_tokens, m.d_step, m.token_cap};
+        if (st.one) {
+        } else if (S == 1 || (cnt == c.batch && (c.batch > 1 || m.sel_first == S - 1))) {
             note(m, adv.ids ? "argmax_advance" : "argmax_last", (double)c.batch * V * 4);
             TRY(argmax_rows<float>(m.d_next, lg, c.batch, V, adv, m.stream));
         } else if (c.batch > 1 || m.sel_first + cnt == S) {

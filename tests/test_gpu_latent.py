@@ -379,7 +379,7 @@ def test_step_profile_names_its_launches(tmp_path):
     # embedding + 4 layer runs of 7 launches + 2 pass starts + head + greedy token
     assert dec.stats() == dict(dec.stats(), launches_per_step=1 + 4 * 7 + 2 + 2, graph=True)
     names = [n for n, ms, _, _ in dec.profile_step(3, 0) if ms > 0]
-    assert names.count("latent_attention") == 4 and names.count("gemv_loop_in") == 2 and names[-1] == "argmax_advance"
+    assert names.count("latent_attention") == 4 and names.count("gemv_loop_in") == 2 and names[-1] == "greedy_advance"
     dec.close()
 
 
