@@ -812,11 +812,14 @@ LATENT_SIZES = {
     "3072": dict(width=3072, heads=24, ff=8192, vocab=64000),
     "4096": dict(width=4096, heads=32, ff=14336, vocab=128256),
 }
-# launch of the design -> the like launch of the Llama graph
+# launch of the design -> the like launch of the Llama graph.  The design's decode attention is three launches -- the queries
+# taken into the latent space, the scores and sums over the cached rows, W_uv and gate -- where the Llama graph has one:
+# "attention_block" is their bytes over their time.
+LATENT_ATTENTION_BLOCK = ("latent_absorb_append", "latent_attention", "latent_merge_out", "attention_rope_append", "rope_kv_append", "attention")
 LATENT_PAIRS = {
     "decode": {"gemv_norm_latent_in": "gemv_norm_qkv", "latent_attention": "attention_rope_append|attention", "gemv_o": "gemv_o_residual",
                "gemv_norm_gateup_geglu": "gemv_norm_gateup_swiglu", "gemv_down": "gemv_down_residual", "gemv_loop_in": "gemv_norm_qkv",
-               "latent_absorb_append": "rope_kv_append", "latent_merge_out": "gemv_o_residual", "gemv_norm_head": "gemv_norm_lm_head"},
+               "attention_block": "attention_block", "gemv_norm_head": "gemv_norm_lm_head"},
     "prefill": {"linear_latent_in": "linear_qkv", "linear_latent_kv": "linear_qkv", "latent_attention": "attention", "linear_o": "linear_o_residual",
                 "linear_gateup_geglu": "linear_gateup_swiglu", "linear_down": "linear_down_residual", "linear_loop_in": "linear_o_residual",
                 "residual_norm": "rms_norm", "residual_concat": "rms_norm", "latent_rotate_append": "rope_kv_append|rope_kv_append_k_v",
@@ -842,7 +845,8 @@ def latent_main(args, mynn):
     import torch
 
     ctx, K, W = 2048, args.steps or 64, args.warmup or 16
-    max_seq, runs = 2560, 6
+    far, runs = 16384, 6  # a second, longer context for the decode launches (cache rows of zeros behind the prompt)
+    max_seq = far + 256
     gen = torch.Generator(device="cuda")
     gen.manual_seed(args.seed)
     rng = np.random.default_rng(args.seed)
@@ -857,6 +861,9 @@ def latent_main(args, mynn):
                 a[2] += nbytes + kv_bytes.get(name, 0.0)
                 a[3] += flops
         out = {}
+        block = [v for k, v in agg.items() if k in LATENT_ATTENTION_BLOCK]
+        if kv_bytes:
+            agg["attention_block"] = [max(v[0] for v in block)] + [sum(v[i] for v in block) for i in (1, 2, 3)]
         for name, (n, ms, nb, fl) in agg.items():
             t = ms * 1e-3
             if t <= 0:
@@ -898,7 +905,10 @@ def latent_main(args, mynn):
         row = (512 + 64) * 2.0  # cached bytes of a token and layer run
         res["latent"] = {"prefill_tok_s": round(ctx / t_pre), "decode_tok_s": round(1 / t_dec, 1), "launches_per_step": dec.stats()["launches_per_step"],
                          "prefill": per_kernel(lambda: pre.profile(ids, pos, 0, ctx), 3, {}),
-                         "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, {"latent_attention": (ctx + 33) * row})}
+                         "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, {"latent_attention": (ctx + 33) * row}),
+                         "decode_far": per_kernel(lambda: dec.profile_step(1, far + 32), 8, {"latent_attention": (far + 33) * row})}
+        dec.decode_loop(1, far, W)
+        res["latent"]["decode_far_tok_s"] = round(K / rate(lambda: dec.decode_loop(1, far, K), 3, 1), 1)
         pre.close(), dec.close()
         del w, state
         # ---- the Llama graph
@@ -911,15 +921,18 @@ def latent_main(args, mynn):
         t_pre = rate(lambda: pre.step(ids, pos, 0, ctx), 5, 2)
         dec.decode_loop(1, ctx, W)
         t_dec = rate(lambda: dec.decode_loop(1, ctx, K), 3, 1) / K
-        kv = (ctx + 33) * 2.0 * cfg["n_kv_heads"] * 128 * 2
+        kv = lambda n: {k: (n + 33) * 2.0 * cfg["n_kv_heads"] * 128 * 2 for k in ("attention_rope_append", "attention")}
         res["llama"] = {"prefill_tok_s": round(ctx / t_pre), "decode_tok_s": round(1 / t_dec, 1), "launches_per_step": dec.stats()["launches_per_step"],
                         "prefill": per_kernel(lambda: pre.profile(ids, pos, 0, ctx), 3, {}),
-                        "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, {"attention_rope_append": kv, "attention": kv})}
+                        "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, kv(ctx)),
+                        "decode_far": per_kernel(lambda: dec.profile_step(1, far + 32), 8, kv(far))}
+        dec.decode_loop(1, far, W)
+        res["llama"]["decode_far_tok_s"] = round(K / rate(lambda: dec.decode_loop(1, far, K), 3, 1), 1)
         pre.close(), dec.close()
         del lw
         torch.cuda.empty_cache()
         # distance from the roofline relative to the like launch's: 1 / frac against 1 / frac
-        for phase, pairs in LATENT_PAIRS.items():
+        for phase, pairs in list(LATENT_PAIRS.items()) + [("decode_far", LATENT_PAIRS["decode"])]:
             res["times_farther_" + phase] = {}
             for mine, like in pairs.items():
                 other = next((o for o in like.split("|") if o in res["llama"][phase]), None)

@@ -138,7 +138,7 @@ int latent_prepare(const LatentParams &p, bool absorb, int dtype, hipStream_t s)
 
 // ---- absorbed attention -------------------------------------------------------------------------------------------------
 // Key ranges: the active rows are cut into at most nsplit ranges of a multiple of 32 rows, at least kMinRange.
-constexpr int kTile = 32, kMinRange = 64;
+constexpr int kTile = 32, kMinRange = 32;
 __device__ __host__ inline int latent_range(int active, int nsplit) {
     const int r = ((active + nsplit - 1) / nsplit + kTile - 1) / kTile * kTile;
     return r < kMinRange ? kMinRange : r;
@@ -160,7 +160,17 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
     float *Ss = (float *)(Qs + 16 * MT * ldc);
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4;
     const int split = blockIdx.x, r0 = blockIdx.y * 16 * MT, b = blockIdx.z;
-    const int past = *p.d_past, nrows = p.S * d.H;
+    const int nrows = p.S * d.H;
+    // idx / cpr for idx < 8192, cpr <= 128 by a multiplication: div = ceil(2^20 / cpr), so idx * (div * cpr - 2^20) < 2^20
+    auto row_of = [&](int idx) { return (int)(((unsigned)idx * div) >> 20); };
+    // the queries (rows past the end become zeros) are requested before anything waits for the context length
+    U4 qv[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; i++) {
+        const int idx = min(tid + i * 256, 16 * MT * cpr - 1), r = row_of(idx);
+        qv[i] = *(const U4 *)((const T *)p.q_abs + ((size_t)b * nrows + min(r0 + r, nrows - 1)) * lw + (idx - r * cpr) * 8);
+    }
+    const int past = *p.d_past;
     const int range = latent_range(past + p.S, p.nsplit);
     const int last_q = min(r0 + 16 * MT - 1, nrows - 1) / d.H;       // the furthest query of the workgroup
     const int k0 = split * range, k1 = min(min(past + p.S, k0 + range), past + last_q + 1);
@@ -186,8 +196,6 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
     // is asked for one tile ahead of the loads that need it)
     auto page_of = [&](int t) { return table ? table[(k0 + min(t, ntiles - 1) * kTile) >> psh] : 0; };
     U4 pre[NL];
-    // idx / cpr for idx < 8192, cpr <= 128 by a multiplication: div = ceil(2^20 / cpr), so idx * (div * cpr - 2^20) < 2^20
-    auto row_of = [&](int idx) { return (int)(((unsigned)idx * div) >> 20); };
     auto load_tile = [&](int t, int page) {
         const int t0 = k0 + t * kTile;
 #pragma unroll
@@ -202,13 +210,6 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
     if (ntiles) {
         load_tile(0, page_of(0));
         page_next = page_of(1);
-        // queries to LDS (rows past the end: zeros), all of a thread's pieces requested together
-        U4 qv[NQ];
-#pragma unroll
-        for (int i = 0; i < NQ; i++) {
-            const int idx = min(tid + i * 256, 16 * MT * cpr - 1), r = row_of(idx);
-            qv[i] = *(const U4 *)((const T *)p.q_abs + ((size_t)b * nrows + min(r0 + r, nrows - 1)) * lw + (idx - r * cpr) * 8);
-        }
 #pragma unroll
         for (int i = 0; i < NQ; i++) {
             const int idx = tid + i * 256, r = row_of(idx);
@@ -454,18 +455,27 @@ int latent_attention_absorbed(const LatentParams &p, int dtype, hipStream_t s) {
 }
 
 // ---- merge of the key ranges, W_uv, gate: 32 value dimensions of one (query, head) per workgroup ---------------------
-constexpr int kMaxRanges = 128;
+constexpr int kMaxRanges = 128, kOutThreads = 256;
 template <typename T>
-__global__ __launch_bounds__(256) void latent_out_kernel(LatentParams p) {
+__global__ __launch_bounds__(kOutThreads) void latent_out_kernel(LatentParams p) {
     extern __shared__ __align__(16) char smem[];
     float *o = (float *)smem;  // [rp], then the partial sums
     __shared__ float wgt[kMaxRanges];
     const LatentDims &d = p.d;
+    constexpr int NT = kOutThreads;
     const int h = blockIdx.y, row = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const size_t at = ((size_t)row * d.H + h) * p.nsplit;
-    // ranges that hold a key this row sees
-    const int live = p.nsplit == 1 ? 1 : (*p.d_past + row % p.S) / latent_range(*p.d_past + p.S, p.nsplit) + 1;
-    // this wave's eight rows of W_uv (a latent of up to 512 values: one piece per lane) are on their way first
+    // Requested before the context length is known, so that the loads are one round trip: the ranges' maxima and sums, the
+    // first kAhead ranges of the thread's four latents, and this wave's first eight rows of W_uv (a latent of up to 512
+    // values: one piece per lane).  What lies past the last live range is not used.
+    constexpr int kAhead = 8;
+    const int n4 = d.rp >> 2, ng = NT / min(n4, NT), grp = tid / n4, c4_0 = tid - grp * n4;  // thread = (four latents, every ng-th range)
+    const float *po = p.part_o + at * d.rp;
+    float4 ahead[kAhead];
+    if (grp < ng) {
+#pragma unroll
+        for (int j = 0; j < kAhead; j++) ahead[j] = *(const float4 *)(po + (size_t)min(grp + j * ng, p.nsplit - 1) * d.rp + c4_0 * 4);
+    }
     const int v0 = blockIdx.x * 32 + wave * 8;
     const T *uv = (const T *)p.ukv + ((size_t)d.H * d.dimp + (size_t)h * d.vdimp + v0) * d.rp;
     const bool have = lane * 8 < d.rp;
@@ -473,32 +483,38 @@ __global__ __launch_bounds__(256) void latent_out_kernel(LatentParams p) {
 #pragma unroll
     for (int j = 0; j < 8; j++)
         if (have) wr[j].get(uv + (size_t)j * d.rp + lane * 8);
+    // ranges that hold a key this row sees
+    const int live = p.nsplit == 1 ? 1 : (*p.d_past + row % p.S) / latent_range(*p.d_past + p.S, p.nsplit) + 1;
     if (wave == 0) {
-        float m = -INFINITY;
-        for (int i = lane; i < live; i += 64) m = fmaxf(m, p.part_ml[(at + i) * 2]);
+        const float *ml = p.part_ml + at * 2;
+        float m = -INFINITY, l = 0.f;
+        for (int i = lane; i < live; i += 64) m = fmaxf(m, ml[2 * i]);
         m = wave_max(m);
-        float l = 0.f;
-        for (int i = lane; i < live; i += 64) l += p.part_ml[(at + i) * 2 + 1] * expf(p.part_ml[(at + i) * 2] - m);
+        for (int i = lane; i < live; i += 64) l += ml[2 * i + 1] * expf(ml[2 * i] - m);
         l = wave_sum(l);
-        for (int i = lane; i < live; i += 64) wgt[i] = expf(p.part_ml[(at + i) * 2] - m) / l;
+        for (int i = lane; i < live; i += 64) wgt[i] = expf(ml[2 * i] - m) / l;
     }
     __syncthreads();
-    // thread = (four latents, every ng-th range), the groups' sums meet in LDS; eight ranges in flight per thread
-    const int n4 = d.rp >> 2, ng = 256 / min(n4, 256), grp = tid / n4;
     float *acc_s = o + d.rp;  // [ng][rp]
-    for (int c4 = tid - grp * n4; c4 < n4 && grp < ng; c4 += 256) {
+    for (int c4 = c4_0; c4 < n4 && grp < ng; c4 += NT) {
         float4 a = float4{0.f, 0.f, 0.f, 0.f};
-        const float *src = p.part_o + at * d.rp + c4 * 4;
-#pragma unroll 8
-        for (int i = grp; i < live; i += ng) {
-            const float4 v = *(const float4 *)(src + (size_t)i * d.rp);
-            const float w = wgt[i];
-            a.x = fmaf(w, v.x, a.x); a.y = fmaf(w, v.y, a.y); a.z = fmaf(w, v.z, a.z); a.w = fmaf(w, v.w, a.w);
+        for (int i0 = grp; i0 < live; i0 += kAhead * ng) {
+            if (i0 != grp || c4 != c4_0) {
+#pragma unroll
+                for (int j = 0; j < kAhead; j++) ahead[j] = *(const float4 *)(po + (size_t)min(i0 + j * ng, live - 1) * d.rp + c4 * 4);
+            }
+#pragma unroll
+            for (int j = 0; j < kAhead; j++)
+                if (i0 + j * ng < live) {
+                    const float w = wgt[i0 + j * ng];
+                    a.x = fmaf(w, ahead[j].x, a.x); a.y = fmaf(w, ahead[j].y, a.y);
+                    a.z = fmaf(w, ahead[j].z, a.z); a.w = fmaf(w, ahead[j].w, a.w);
+                }
         }
         *(float4 *)(acc_s + grp * d.rp + c4 * 4) = a;
     }
     __syncthreads();
-    for (int k = tid; k < d.rp; k += 256) {
+    for (int k = tid; k < d.rp; k += NT) {
         float a = 0.f;
         for (int i = 0; i < ng; i++) a += acc_s[i * d.rp + k];
         o[k] = a;
@@ -527,13 +543,12 @@ __global__ __launch_bounds__(256) void latent_out_kernel(LatentParams p) {
 int latent_merge_out(const LatentParams &p, int dtype, hipStream_t s) {
     MYNN_REQUIRE(p.out && p.part_o && p.part_ml && p.ukv && p.proj && p.nsplit >= 1 && p.nsplit <= kMaxRanges, MYNN_ERR_INVALID, "latent merge: bad operand");
     MYNN_REQUIRE(p.B * p.S <= 65535, MYNN_ERR_UNSUPPORTED, "latent merge: %d rows", p.B * p.S);
-    const dim3 grid(p.d.vdimp / 32, p.d.H, p.B * p.S);
+    const int nt = kOutThreads;
+    const size_t lds = (size_t)(1 + nt / std::min(p.d.rp >> 2, nt)) * p.d.rp * 4;
+    MYNN_REQUIRE(lds <= 60 * 1024, MYNN_ERR_UNSUPPORTED, "latent merge: latent of %d values", p.d.rank);
     return dispatch_dense(dtype, [&](auto *t) {
         using T = std::remove_pointer_t<decltype(t)>;
-        const int ng = 256 / std::min(p.d.rp >> 2, 256);
-        const size_t lds = (size_t)(1 + ng) * p.d.rp * 4;
-        MYNN_REQUIRE(lds <= 60 * 1024, MYNN_ERR_UNSUPPORTED, "latent merge: latent of %d values", p.d.rank);
-        MYNN_LAUNCH(latent_out_kernel<T>, grid, dim3(256), lds, s, p);
+        MYNN_LAUNCH(latent_out_kernel<T>, dim3(p.d.vdimp / 32, p.d.H, p.B * p.S), dim3(nt), lds, s, p);
         return launch_status("latent_out_kernel");
     });
 }
