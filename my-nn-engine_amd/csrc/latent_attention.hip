@@ -137,22 +137,24 @@ int latent_prepare(const LatentParams &p, bool absorb, int dtype, hipStream_t s)
 }
 
 // ---- absorbed attention -------------------------------------------------------------------------------------------------
-// Key ranges: the active rows are cut into at most nsplit ranges of a multiple of 32 rows, at least kMinRange.
-constexpr int kTile = 32, kMinRange = 32;
+// Key ranges: the active rows are cut into at most nsplit ranges of a multiple of 64 rows.
+constexpr int kTile = 64, kMinRange = 64;
 __device__ __host__ inline int latent_range(int active, int nsplit) {
     const int r = ((active + nsplit - 1) / nsplit + kTile - 1) / kTile * kTile;
     return r < kMinRange ? kMinRange : r;
 }
 
-// One workgroup: 16 * MT rows of a sequence's (query, head) pairs against one key range.  Tiles of 32 keys: the tile is
-// staged in LDS (the next one waits in registers), the four waves share the score product (by key half and by query tile,
-// or by halves of the row for MT == 1), every wave then takes the softmax of all rows and adds its own 32-column blocks
-// of P . C.  CB: 32-column blocks per wave.
+// One workgroup of eight waves: 16 * MT rows of a sequence's (query, head) pairs against one key range.  Tiles of 64 keys:
+// the tile is staged in LDS (the next one waits in registers), the waves share the score product (by 16 keys and by query
+// tile, or by halves of the row for MT == 1), every wave then takes the softmax of all rows and adds its own 32-column
+// blocks of P . C.  CB: 32-column blocks per wave.  div: ceil(2^20 / (16-byte pieces of a row)).
+constexpr int kAbsThreads = 512, kAbsWaves = kAbsThreads / 64;
 template <typename T, int MT, int CB>
-__global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, unsigned div) {
-    constexpr int KS = MT == 1 ? 2 : 1;  // partial score products per (key, query)
-    constexpr int NL = 2 * CB + 2, NQ = MT * (CB + 1);  // 16-byte pieces of a tile / of the queries per thread
+__global__ __launch_bounds__(kAbsThreads) void latent_absorbed_kernel(LatentParams p, unsigned div) {
+    constexpr int KS = MT == 1 ? 2 : 1;                     // partial score products per (key, query)
+    constexpr int NL = 4 * CB + 2, NQ = MT * (CB + 1);      // 16-byte pieces of a tile / of the queries per thread
     constexpr int SST = kTile + 4;
+    static_assert(kTile == 64 && kAbsWaves == 8, "four key groups of 16, two score products each");
     extern __shared__ __align__(16) char smem[];
     const LatentDims &d = p.d;
     const int lw = d.lw(), ldc = lw + 8, cpr = lw >> 3;
@@ -161,23 +163,22 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4;
     const int split = blockIdx.x, r0 = blockIdx.y * 16 * MT, b = blockIdx.z;
     const int nrows = p.S * d.H;
-    // idx / cpr for idx < 8192, cpr <= 128 by a multiplication: div = ceil(2^20 / cpr), so idx * (div * cpr - 2^20) < 2^20
+    // idx / cpr for idx < 8192, cpr <= 128 by a multiplication (idx * (div * cpr - 2^20) < 2^20)
     auto row_of = [&](int idx) { return (int)(((unsigned)idx * div) >> 20); };
     // the queries (rows past the end become zeros) are requested before anything waits for the context length
     U4 qv[NQ];
 #pragma unroll
     for (int i = 0; i < NQ; i++) {
-        const int idx = min(tid + i * 256, 16 * MT * cpr - 1), r = row_of(idx);
+        const int idx = min(tid + i * kAbsThreads, 16 * MT * cpr - 1), r = row_of(idx);
         qv[i] = *(const U4 *)((const T *)p.q_abs + ((size_t)b * nrows + min(r0 + r, nrows - 1)) * lw + (idx - r * cpr) * 8);
     }
     const int past = *p.d_past;
     const int range = latent_range(past + p.S, p.nsplit);
     const int last_q = min(r0 + 16 * MT - 1, nrows - 1) / d.H;       // the furthest query of the workgroup
     const int k0 = split * range, k1 = min(min(past + p.S, k0 + range), past + last_q + 1);
-
     int bound[MT];  // keys the row of this lane's column sees
 #pragma unroll
-    for (int m = 0; m < MT; m++) bound[m] = past + min(r0 + 16 * m + col, nrows - 1) / d.H + 1;
+    for (int m = 0; m < MT; m++) bound[m] = min(past + min(r0 + 16 * m + col, nrows - 1) / d.H + 1, k1);
 
     float m_run[MT], l_run[MT];
     lf4_t acc[MT][CB][2];
@@ -192,7 +193,7 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
     const int psh = p.paging.shift, pmask = (1 << psh) - 1;
     const int32_t *table = p.paging.table ? p.paging.table + (size_t)b * p.paging.pages_per_seq : nullptr;
     const int ntiles = k1 > k0 ? (k1 - k0 + kTile - 1) / kTile : 0;
-    // (a tile starts at a multiple of 32 and a page holds a multiple of 32 rows: a tile lies in one page, whose number
+    // (a tile starts at a multiple of 64 and a page holds a multiple of 64 rows: a tile lies in one page, whose number
     // is asked for one tile ahead of the loads that need it)
     auto page_of = [&](int t) { return table ? table[(k0 + min(t, ntiles - 1) * kTile) >> psh] : 0; };
     U4 pre[NL];
@@ -200,7 +201,7 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
         const int t0 = k0 + t * kTile;
 #pragma unroll
         for (int i = 0; i < NL; i++) {
-            const int idx = min(tid + i * 256, kTile * cpr - 1), r = row_of(idx);
+            const int idx = min(tid + i * kAbsThreads, kTile * cpr - 1), r = row_of(idx);
             const int key = min(t0 + r, k1 - 1);
             const size_t row = table ? ((size_t)page << psh) + (key & pmask) : (size_t)b * p.max_seq + key;
             pre[i] = *(const U4 *)((const T *)p.cache + row * lw + (idx - r * cpr) * 8);
@@ -212,7 +213,7 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
         page_next = page_of(1);
 #pragma unroll
         for (int i = 0; i < NQ; i++) {
-            const int idx = tid + i * 256, r = row_of(idx);
+            const int idx = tid + i * kAbsThreads, r = row_of(idx);
             if (idx < 16 * MT * cpr) *(U4 *)(Qs + r * ldc + (idx - r * cpr) * 8) = r0 + r < nrows ? qv[i] : U4{0u, 0u, 0u, 0u};
         }
     }
@@ -221,7 +222,7 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
         __syncthreads();  // the tile before is no longer read
 #pragma unroll
         for (int i = 0; i < NL; i++) {
-            const int idx = tid + i * 256, r = row_of(idx);
+            const int idx = tid + i * kAbsThreads, r = row_of(idx);
             if (idx < kTile * cpr) *(U4 *)(Cs + r * ldc + (idx - r * cpr) * 8) = pre[i];
         }
         __syncthreads();
@@ -231,7 +232,7 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
         }
         // ---- scores: this wave's 16 keys x 16 rows
         {
-            const int kt = wave & 1, other = wave >> 1;
+            const int kt = wave & 3, other = wave >> 2;
             const int qt = MT == 1 ? 0 : other;
             lf4_t s4 = {0.f, 0.f, 0.f, 0.f}, s5 = {0.f, 0.f, 0.f, 0.f};
             const T *ca = Cs + (kt * 16 + col) * ldc + quad * 8, *qb = Qs + (qt * 16 + col) * ldc + quad * 8;
@@ -255,26 +256,29 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
             *(float4 *)dst = float4{s4[0], s4[1], s4[2], s4[3]};
         }
         __syncthreads();
-        // ---- softmax of row `col` of every query tile, keys 8 * quad .. + 7 of the tile
+        // ---- softmax of row `col` of every query tile, keys 32 * half + 8 * quad .. + 7 of the tile
         const int key0 = k0 + t * kTile + quad * 8;
-        U4 ph[MT], pl[MT];
+        U4 ph[MT][2], pl[MT][2];
 #pragma unroll
         for (int m = 0; m < MT; m++) {
-            float sv[8];
-            const float *src = Ss + (m * 16 + col) * SST + quad * 8;
-            *(float4 *)sv = *(const float4 *)src;
-            *(float4 *)(sv + 4) = *(const float4 *)(src + 4);
-            if constexpr (KS == 2) {
-                const float4 a = *(const float4 *)(src + 16 * MT * SST), c = *(const float4 *)(src + 16 * MT * SST + 4);
-                sv[0] += a.x; sv[1] += a.y; sv[2] += a.z; sv[3] += a.w;
-                sv[4] += c.x; sv[5] += c.y; sv[6] += c.z; sv[7] += c.w;
-            }
+            float sv[16];
             float tmax = -INFINITY;
-            const int lim = min(bound[m], k1);
 #pragma unroll
-            for (int e = 0; e < 8; e++) {
-                sv[e] = key0 + e < lim ? sv[e] * p.scale : -INFINITY;
-                tmax = fmaxf(tmax, sv[e]);
+            for (int hf = 0; hf < 2; hf++) {
+                const float *src = Ss + (m * 16 + col) * SST + hf * 32 + quad * 8;
+                float *v = sv + 8 * hf;
+                *(float4 *)v = *(const float4 *)src;
+                *(float4 *)(v + 4) = *(const float4 *)(src + 4);
+                if constexpr (KS == 2) {
+                    const float4 a = *(const float4 *)(src + 16 * MT * SST), c = *(const float4 *)(src + 16 * MT * SST + 4);
+                    v[0] += a.x; v[1] += a.y; v[2] += a.z; v[3] += a.w;
+                    v[4] += c.x; v[5] += c.y; v[6] += c.z; v[7] += c.w;
+                }
+#pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    v[e] = key0 + 32 * hf + e < bound[m] ? v[e] * p.scale : -INFINITY;
+                    tmax = fmaxf(tmax, v[e]);
+                }
             }
             tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
             tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
@@ -283,13 +287,13 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
             if (m_new > -INFINITY) {
                 alpha = fast_exp(m_run[m] - m_new);
 #pragma unroll
-                for (int e = 0; e < 8; e++) {
+                for (int e = 0; e < 16; e++) {
                     sv[e] = fast_exp(sv[e] - m_new);
                     psum += sv[e];
                 }
             } else {
 #pragma unroll
-                for (int e = 0; e < 8; e++) sv[e] = 0.f;
+                for (int e = 0; e < 16; e++) sv[e] = 0.f;
             }
             m_run[m] = m_new;
             l_run[m] = l_run[m] * alpha + psum;
@@ -301,31 +305,38 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
                 }
             }
             // the weights enter the product as a sum of two storage-type values
-            ph[m] = U4{pack2<T>(sv[0], sv[1]), pack2<T>(sv[2], sv[3]), pack2<T>(sv[4], sv[5]), pack2<T>(sv[6], sv[7])};
-            float hi[8];
-            widen8<T>(ph[m], hi);
 #pragma unroll
-            for (int e = 0; e < 8; e++) sv[e] -= hi[e];
-            pl[m] = U4{pack2<T>(sv[0], sv[1]), pack2<T>(sv[2], sv[3]), pack2<T>(sv[4], sv[5]), pack2<T>(sv[6], sv[7])};
+            for (int hf = 0; hf < 2; hf++) {
+                float *v = sv + 8 * hf;
+                ph[m][hf] = U4{pack2<T>(v[0], v[1]), pack2<T>(v[2], v[3]), pack2<T>(v[4], v[5]), pack2<T>(v[6], v[7])};
+                float hi[8];
+                widen8<T>(ph[m][hf], hi);
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] -= hi[e];
+                pl[m][hf] = U4{pack2<T>(v[0], v[1]), pack2<T>(v[2], v[3]), pack2<T>(v[4], v[5]), pack2<T>(v[6], v[7])};
+            }
         }
         // ---- O^T += C^T . P: a pair of neighbouring latents per dword, split into two operands by v_perm
 #pragma unroll
         for (int c = 0; c < CB; c++) {
-            const int blk = wave + 4 * c;
+            const int blk = wave + kAbsWaves * c;
             if (blk < nblk) {
-                uint32_t w[8];
 #pragma unroll
-                for (int i = 0; i < 8; i++) w[i] = *(const uint32_t *)(Cs + (quad * 8 + i) * ldc + blk * 32 + col * 2);
-                const U4 ev = U4{__builtin_amdgcn_perm(w[1], w[0], 0x05040100u), __builtin_amdgcn_perm(w[3], w[2], 0x05040100u),
-                                 __builtin_amdgcn_perm(w[5], w[4], 0x05040100u), __builtin_amdgcn_perm(w[7], w[6], 0x05040100u)};
-                const U4 od = U4{__builtin_amdgcn_perm(w[1], w[0], 0x07060302u), __builtin_amdgcn_perm(w[3], w[2], 0x07060302u),
-                                 __builtin_amdgcn_perm(w[5], w[4], 0x07060302u), __builtin_amdgcn_perm(w[7], w[6], 0x07060302u)};
+                for (int hf = 0; hf < 2; hf++) {
+                    uint32_t w[8];
 #pragma unroll
-                for (int m = 0; m < MT; m++) {
-                    acc[m][c][0] = MfmaL16<T>::run(ev, ph[m], acc[m][c][0]);
-                    acc[m][c][1] = MfmaL16<T>::run(od, ph[m], acc[m][c][1]);
-                    acc[m][c][0] = MfmaL16<T>::run(ev, pl[m], acc[m][c][0]);
-                    acc[m][c][1] = MfmaL16<T>::run(od, pl[m], acc[m][c][1]);
+                    for (int i = 0; i < 8; i++) w[i] = *(const uint32_t *)(Cs + (hf * 32 + quad * 8 + i) * ldc + blk * 32 + col * 2);
+                    const U4 ev = U4{__builtin_amdgcn_perm(w[1], w[0], 0x05040100u), __builtin_amdgcn_perm(w[3], w[2], 0x05040100u),
+                                     __builtin_amdgcn_perm(w[5], w[4], 0x05040100u), __builtin_amdgcn_perm(w[7], w[6], 0x05040100u)};
+                    const U4 od = U4{__builtin_amdgcn_perm(w[1], w[0], 0x07060302u), __builtin_amdgcn_perm(w[3], w[2], 0x07060302u),
+                                     __builtin_amdgcn_perm(w[5], w[4], 0x07060302u), __builtin_amdgcn_perm(w[7], w[6], 0x07060302u)};
+#pragma unroll
+                    for (int m = 0; m < MT; m++) {
+                        acc[m][c][0] = MfmaL16<T>::run(ev, ph[m][hf], acc[m][c][0]);
+                        acc[m][c][1] = MfmaL16<T>::run(od, ph[m][hf], acc[m][c][1]);
+                        acc[m][c][0] = MfmaL16<T>::run(ev, pl[m][hf], acc[m][c][0]);
+                        acc[m][c][1] = MfmaL16<T>::run(od, pl[m][hf], acc[m][c][1]);
+                    }
                 }
             }
         }
@@ -340,7 +351,7 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(LatentParams p, un
         const size_t at = ((size_t)b * nrows + r) * p.nsplit + split;
 #pragma unroll
         for (int c = 0; c < CB; c++) {
-            const int blk = wave + 4 * c;
+            const int blk = wave + kAbsWaves * c;
             if (blk < nblk) {
                 float *dst = p.part_o + at * d.rp + blk * 32 + 8 * quad;
                 *(float4 *)dst = float4{acc[m][c][0][0], acc[m][c][1][0], acc[m][c][0][1], acc[m][c][1][1]};
@@ -446,23 +457,22 @@ int latent_attention_absorbed(const LatentParams &p, int dtype, hipStream_t s) {
     const size_t lds = (size_t)(kTile + 16 * mt) * (d.lw() + 8) * 2 + (size_t)(mt == 1 ? 2 : 1) * 16 * mt * (kTile + 4) * 4;
     auto go = [&](auto kernel) {
         if (lds > 60 * 1024) MYNN_HIP(hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-        MYNN_LAUNCH(kernel, grid, dim3(256), lds, s, p, ((1u << 20) + cpr - 1) / cpr);
+        MYNN_LAUNCH(kernel, grid, dim3(kAbsThreads), lds, s, p, ((1u << 20) + cpr - 1) / cpr);
         return launch_status("latent_absorbed_kernel");
     };
-    const int nblk = d.rp >> 5;
-    if (mt == 1) return nblk <= 4 ? go(latent_absorbed_kernel<bf16_t, 1, 1>) : nblk <= 8 ? go(latent_absorbed_kernel<bf16_t, 1, 2>) : go(latent_absorbed_kernel<bf16_t, 1, 4>);
-    return nblk <= 4 ? go(latent_absorbed_kernel<bf16_t, 2, 1>) : nblk <= 8 ? go(latent_absorbed_kernel<bf16_t, 2, 2>) : go(latent_absorbed_kernel<bf16_t, 2, 4>);
+    const bool wide = (d.rp >> 5) > kAbsWaves;
+    if (mt == 1) return wide ? go(latent_absorbed_kernel<bf16_t, 1, 2>) : go(latent_absorbed_kernel<bf16_t, 1, 1>);
+    return wide ? go(latent_absorbed_kernel<bf16_t, 2, 2>) : go(latent_absorbed_kernel<bf16_t, 2, 1>);
 }
 
-// ---- merge of the key ranges, W_uv, gate: 32 value dimensions of one (query, head) per workgroup ---------------------
-constexpr int kMaxRanges = 128, kOutThreads = 256;
-template <typename T>
-__global__ __launch_bounds__(kOutThreads) void latent_out_kernel(LatentParams p) {
+// ---- merge of the key ranges, W_uv, gate: NT / 8 value dimensions of one (query, head) per workgroup -----------------
+constexpr int kMaxRanges = 128;
+template <typename T, int NT>
+__global__ __launch_bounds__(NT) void latent_out_kernel(LatentParams p) {
     extern __shared__ __align__(16) char smem[];
     float *o = (float *)smem;  // [rp], then the partial sums
     __shared__ float wgt[kMaxRanges];
     const LatentDims &d = p.d;
-    constexpr int NT = kOutThreads;
     const int h = blockIdx.y, row = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const size_t at = ((size_t)row * d.H + h) * p.nsplit;
     // Requested before the context length is known, so that the loads are one round trip: the ranges' maxima and sums, the
@@ -470,13 +480,18 @@ __global__ __launch_bounds__(kOutThreads) void latent_out_kernel(LatentParams p)
     // values: one piece per lane).  What lies past the last live range is not used.
     constexpr int kAhead = 8;
     const int n4 = d.rp >> 2, ng = NT / min(n4, NT), grp = tid / n4, c4_0 = tid - grp * n4;  // thread = (four latents, every ng-th range)
-    const float *po = p.part_o + at * d.rp;
+    const float *po = p.part_o + at * d.rp, *ml = p.part_ml + at * 2;
+    float2 r_ml[kMaxRanges / 64];
+    if (wave == 0) {
+#pragma unroll
+        for (int i = 0; i < kMaxRanges / 64; i++) r_ml[i] = *(const float2 *)(ml + 2 * min(lane + 64 * i, p.nsplit - 1));
+    }
     float4 ahead[kAhead];
     if (grp < ng) {
 #pragma unroll
         for (int j = 0; j < kAhead; j++) ahead[j] = *(const float4 *)(po + (size_t)min(grp + j * ng, p.nsplit - 1) * d.rp + c4_0 * 4);
     }
-    const int v0 = blockIdx.x * 32 + wave * 8;
+    const int v0 = blockIdx.x * (NT / 8) + wave * 8;
     const T *uv = (const T *)p.ukv + ((size_t)d.H * d.dimp + (size_t)h * d.vdimp + v0) * d.rp;
     const bool have = lane * 8 < d.rp;
     Row8<T> wr[8];
@@ -486,13 +501,19 @@ __global__ __launch_bounds__(kOutThreads) void latent_out_kernel(LatentParams p)
     // ranges that hold a key this row sees
     const int live = p.nsplit == 1 ? 1 : (*p.d_past + row % p.S) / latent_range(*p.d_past + p.S, p.nsplit) + 1;
     if (wave == 0) {
-        const float *ml = p.part_ml + at * 2;
-        float m = -INFINITY, l = 0.f;
-        for (int i = lane; i < live; i += 64) m = fmaxf(m, ml[2 * i]);
+        float m = -INFINITY, l = 0.f, e[kMaxRanges / 64];
+#pragma unroll
+        for (int i = 0; i < kMaxRanges / 64; i++)
+            if (lane + 64 * i < live) m = fmaxf(m, r_ml[i].x);
         m = wave_max(m);
-        for (int i = lane; i < live; i += 64) l += ml[2 * i + 1] * expf(ml[2 * i] - m);
+#pragma unroll
+        for (int i = 0; i < kMaxRanges / 64; i++) {
+            e[i] = lane + 64 * i < live ? expf(r_ml[i].x - m) : 0.f;
+            l += lane + 64 * i < live ? e[i] * r_ml[i].y : 0.f;
+        }
         l = wave_sum(l);
-        for (int i = lane; i < live; i += 64) wgt[i] = expf(ml[2 * i] - m) / l;
+#pragma unroll
+        for (int i = 0; i < kMaxRanges / 64; i++) wgt[lane + 64 * i] = e[i] / l;
     }
     __syncthreads();
     float *acc_s = o + d.rp;  // [ng][rp]
@@ -543,12 +564,14 @@ __global__ __launch_bounds__(kOutThreads) void latent_out_kernel(LatentParams p)
 int latent_merge_out(const LatentParams &p, int dtype, hipStream_t s) {
     MYNN_REQUIRE(p.out && p.part_o && p.part_ml && p.ukv && p.proj && p.nsplit >= 1 && p.nsplit <= kMaxRanges, MYNN_ERR_INVALID, "latent merge: bad operand");
     MYNN_REQUIRE(p.B * p.S <= 65535, MYNN_ERR_UNSUPPORTED, "latent merge: %d rows", p.B * p.S);
-    const int nt = kOutThreads;
+    const int nt = p.d.vdimp % 64 ? 256 : 512;
     const size_t lds = (size_t)(1 + nt / std::min(p.d.rp >> 2, nt)) * p.d.rp * 4;
     MYNN_REQUIRE(lds <= 60 * 1024, MYNN_ERR_UNSUPPORTED, "latent merge: latent of %d values", p.d.rank);
     return dispatch_dense(dtype, [&](auto *t) {
         using T = std::remove_pointer_t<decltype(t)>;
-        MYNN_LAUNCH(latent_out_kernel<T>, dim3(p.d.vdimp / 32, p.d.H, p.B * p.S), dim3(nt), lds, s, p);
+        const dim3 grid(p.d.vdimp / (nt / 8), p.d.H, p.B * p.S);
+        if (nt == 512) MYNN_LAUNCH((latent_out_kernel<T, 512>), grid, dim3(512), lds, s, p);
+        else MYNN_LAUNCH((latent_out_kernel<T, 256>), grid, dim3(256), lds, s, p);
         return launch_status("latent_out_kernel");
     });
 }
