@@ -48,23 +48,21 @@ template <typename T> __global__ __launch_bounds__(256) void embed_tokens_kernel
         const int64_t prev = s > 0 ? in_vocab(p.ids[row - 1]) : (int64_t)p.history[history_row(p, b, pos - 1)];
         pair_row = (prev * p.mul_prev + id * p.mul_cur) % p.buckets;
     }
-    if (threadIdx.x == 0) p.history[history_row(p, b, pos)] = (int32_t)id;
-    const T *e = (const T *)p.table + (size_t)id * p.width;
-    const T *pr = p.buckets ? (const T *)p.pair + (size_t)pair_row * p.width : nullptr;
-    for (int k = threadIdx.x; k < p.ld; k += 256) {
-        float v = 0.f;
-        if (k < p.width) {
-            v = Elem<T>::ld(e, k);
-            if (pr) v += Elem<T>::ld(pr, k);
-        }
-        p.x[(size_t)row * p.ld + k] = v;
-        if (p.x0) p.x0[(size_t)row * p.ld + k] = v;
+    const int k = blockIdx.y * 256 + threadIdx.x;
+    if (k == 0) p.history[history_row(p, b, pos)] = (int32_t)id;
+    if (k >= p.ld) return;
+    float v = 0.f;
+    if (k < p.width) {
+        v = Elem<T>::ld((const T *)p.table, (size_t)id * p.width + k);
+        if (p.buckets) v += Elem<T>::ld((const T *)p.pair, (size_t)pair_row * p.width + k);
     }
+    p.x[(size_t)row * p.ld + k] = v;
+    if (p.x0) p.x0[(size_t)row * p.ld + k] = v;
 }
 int embed_tokens(const EmbedParams &p, int dtype, hipStream_t s) {
     return dispatch_dense(dtype, [&](auto *t) {
         using T = std::remove_pointer_t<decltype(t)>;
-        MYNN_LAUNCH(embed_tokens_kernel<T>, dim3(p.B * p.S), dim3(256), 0, s, p);
+        MYNN_LAUNCH(embed_tokens_kernel<T>, dim3(p.B * p.S, (p.ld + 255) / 256), dim3(256), 0, s, p);
         return launch_status("embed_tokens_kernel");
     });
 }
