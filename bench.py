@@ -832,7 +832,7 @@ def latent_config(size):
     mix = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
     layer = {"type": "latent_attention", "mixer": mix, "mlp": {"kind": "dense", "ff": size["ff"]}}
     return {"architecture": "Dudilix", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-5}, "logit_scale": 1.0,
-            "embedding": {"bigram": {"buckets": 4096, "mul_prev": 127, "mul_cur": 31}}, "layers": [layer] * 4,
+            "embedding": {"bigram": {"buckets": 4096, "mul_prev": 131, "mul_cur": 29}}, "layers": [layer] * 4,
             "loop": {"start": 1, "stop": 3, "times": 2}}
 
 

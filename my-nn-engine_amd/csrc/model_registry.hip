@@ -114,8 +114,8 @@ static void read_dudilix(const Reader &r, ModelSpec &s) {
         if (e.has("bigram")) {
             const Reader b = e.sub("bigram");
             s.bigram.buckets = b.integer("buckets", 1, 1 << 28);
-            s.bigram.mul_prev = b.integer("mul_prev", 0, (int64_t)1 << 31);
-            s.bigram.mul_cur = b.integer("mul_cur", 0, (int64_t)1 << 31);
+            s.bigram.mul_prev = b.integer("mul_prev", 0, (int64_t)1 << 32);
+            s.bigram.mul_cur = b.integer("mul_cur", 0, (int64_t)1 << 32);
         }
     }
     const Json *layers = r.need("layers", Json::ARR);

@@ -23,11 +23,11 @@ DTYPES = [pytest.param(F32, id="f32"), pytest.param(BF16, id="bf16")]
 MODELS = {
     "odd": L.config(100, 333, [(L.mixer(3, 24, 8, 16, 40), 70), (L.mixer(2, 32, 4, 48, 100), None), (L.mixer(1, 16, 16, 32, 8), 36)],
                     loop=(1, 3, 3), bigram=(77, 31, 5), eps=1e-3, logit_scale=3.5),
-    "plain": L.config(128, 256, [(L.mixer(2, 64, 32, 64, 128, base=500000.0), 192)] * 2),
+    "plain": L.config(128, 256, [(L.mixer(2, 64, 32, 64, 128, base=250000.0), 192)] * 2),
     "all_looped": L.config(72, 150, [(L.mixer(5, 40, 24, 24, 72), 96), (L.mixer(5, 40, 24, 24, 72), 50)], loop=(0, 2, 2), bigram=(11, 7, 3)),
     "wide_latent": L.config(160, 200, [(L.mixer(4, 128, 64, 128, 320, scale=0.02), 130)], bigram=(1, 1, 1)),
     "many_heads": L.config(192, 500, [(L.mixer(20, 16, 6, 80, 136, rot_dims=4), None), (L.mixer(20, 16, 6, 80, 136), 64)], loop=(1, 2, 2)),
-    "one_pass_loop": L.config(64, 97, [(L.mixer(1, 8, 2, 8, 16), 24)] * 2, loop=(0, 1, 1), bigram=(1000, 127, 509), logit_scale=0.25),
+    "one_pass_loop": L.config(64, 97, [(L.mixer(1, 8, 2, 8, 16), 24)] * 2, loop=(0, 1, 1), bigram=(1000, 113, 401), logit_scale=0.25),
 }
 
 
@@ -172,7 +172,7 @@ def test_loop_passes_have_caches_of_their_own(tmp_path, dt):
 
 # ---- kernel forms -------------------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("heads,dim,rot,vdim,rank", [
-    (2, 64, 16, 64, 64), (3, 100, 28, 64, 130), (1, 192, 64, 33, 64), (2, 32, 32, 128, 256), (4, 128, 64, 128, 512), (1, 160, 32, 100, 64),
+    (2, 64, 24, 56, 64), (3, 100, 28, 64, 130), (1, 192, 64, 33, 64), (2, 32, 32, 128, 256), (4, 128, 64, 128, 512), (1, 160, 32, 100, 64),
     (17, 32, 32, 32, 200), (33, 16, 16, 16, 450), (2, 224, 64, 64, 64), (2, 32, 16, 160, 64), (1, 32, 128, 64, 64), (2, 32, 160, 64, 64), (2, 16, 8, 16, 600)])
 def test_attention_forms(tmp_path, heads, dim, rot, vdim, rank):
     """bf16: every tile form of the prompt and the decode kernels, and the shapes beyond them"""
@@ -305,7 +305,7 @@ def test_sessions_share_pages_and_reuse_them(case, dt):
 @pytest.mark.parametrize("dt", DTYPES)
 def test_rewind_finds_the_previous_token(case, dt):
     toks, other = case.tokens(100), case.tokens(30)
-    eng = mynn.Engine(case.path, dt, 128)
+    eng = mynn.Engine(case.path, dt, 128, page_rows=128)
     s = eng.session()
     s.feed(toks, [])
     s.past_len = 70
