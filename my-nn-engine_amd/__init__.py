@@ -141,6 +141,7 @@ SIGNATURES = {
     "mynn_arch_tensor": (C.c_char_p, [_i, _i, C.POINTER(_i64), C.POINTER(_i)]),
     "mynn_arch_state_count": (_i, [_i]),
     "mynn_arch_state_row_bytes": (_sz, [_i, _i, _i]),
+    "mynn_arch_state_seq_bytes": (_sz, [_i, _i]),
     "mynn_engine_open": (_vp, [C.c_char_p, C.POINTER(EngineOptions)]),
     "mynn_engine_vocab": (_i, [_vp]),
     "mynn_engine_session": (_vp, [_vp, _i64]),
@@ -943,6 +944,10 @@ class Arch:
             out.append((name, tuple(shape[d] for d in range(nd.value))))
         return out
 
+    def state_seq_bytes(self):
+        """bytes per sequence of the state buffers that stand for all tokens read so far (0: a buffer of rows)"""
+        return [lib().mynn_arch_state_seq_bytes(self.id, i) for i in range(lib().mynn_arch_state_count(self.id))]
+
     def state_row_bytes(self, dtype):
         return [lib().mynn_arch_state_row_bytes(self.id, i, dtype) for i in range(lib().mynn_arch_state_count(self.id))]
 
@@ -959,7 +964,7 @@ class LayeredDecoder(object):
         self.arch, self.cfg = arch, arch.config(dtype, max_seq, seq_q, batch)
         self.cfg.kv_page_rows = kv_pages.pool.page_rows if kv_pages is not None else 0
         self.weights, self.kv_pages = weights, kv_pages
-        self.state = state if state is not None else layered_state(arch, dtype, batch * max_seq)
+        self.state = state if state is not None else layered_state(arch, dtype, batch * max_seq, batch=batch)
         ptrs = [t.data_ptr() for t in self.state] + ([kv_pages.handle] if kv_pages is not None else [])
         self._state = (_vp * len(ptrs))(*ptrs)
         self._init = (_vp * len(arch.tensors()))(*[_ptr(weights[n]) for n, _ in arch.tensors()])
@@ -995,11 +1000,12 @@ class LayeredDecoder(object):
         return (list(nxt) if want_next else None), out
 
 
-def layered_state(arch, dtype, rows, fill=0):
-    """Session-state buffers of `rows` cache rows each (batch * max_seq, or n_pages * page_rows of a pool)."""
+def layered_state(arch, dtype, rows, fill=0, batch=1):
+    """Session-state buffers: `rows` cache rows (batch * max_seq, or n_pages * page_rows of a pool), `batch` sequence states."""
     import torch
 
-    return [torch.full((rows * b,), fill, dtype=torch.uint8, device="cuda") for b in arch.state_row_bytes(dtype)]
+    return [torch.full((rows * r + batch * s,), fill, dtype=torch.uint8, device="cuda")
+            for r, s in zip(arch.state_row_bytes(dtype), arch.state_seq_bytes())]
 
 
 class Engine:

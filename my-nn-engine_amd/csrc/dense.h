@@ -27,6 +27,14 @@ struct PackBlocks {
 };
 int pack_blocks(const PackBlocks &p, int dtype, hipStream_t s);
 
+// f32 weights of a short convolution, tap by tap: dst[j * channels + ch0 + h * dimp + i] = src[(h * dim + i) * taps + j]
+struct PackTaps {
+    float *dst;
+    const void *src;
+    int channels, ch0, heads, dim, dimp, taps;
+};
+int pack_taps(const PackTaps &p, int dtype, hipStream_t s);
+
 // x[row] = table[id] (+ pair[hash of (previous id, id)]) as f32 [rows, ld]; row b * S + s is token past + s of sequence b.
 // The ids are recorded in `history` (a cache row per token), where the previous id of a step's first token is found.
 struct EmbedParams {
@@ -42,9 +50,10 @@ struct EmbedParams {
 int embed_tokens(const EmbedParams &p, int dtype, hipStream_t s);
 
 // What precedes a linear: the sublayer output y still to be added to the residual stream, and the norm of the result.
-//   x' = x + rms_norm(y, wb)      (y null: x' = x)
-//   RESIDUAL_NORM: act = rms_norm(x', wa);  RESIDUAL_CONCAT: act = [x', x0];  ROWS: act is a row of T already
-enum { PRO_ROWS = 0, PRO_RESIDUAL_NORM = 1, PRO_RESIDUAL_CONCAT = 2 };
+//   x' = x + y_mul * rms_norm(y, wb)      (y null: x' = x)
+//   RESIDUAL_NORM: act = rms_norm(x', wa);  RESIDUAL_CONCAT: act = [x', x0];  RESIDUAL: act = x';  ROWS: act is a row of T
+//   already.  A norm's weight is w_add + the stored one.
+enum { PRO_ROWS = 0, PRO_RESIDUAL_NORM = 1, PRO_RESIDUAL_CONCAT = 2, PRO_RESIDUAL = 3 };
 struct ResidualNorm {
     const float *x;
     const void *y, *wb;
@@ -53,6 +62,7 @@ struct ResidualNorm {
     const float *x0;
     float eps;
     int width, ld;           // row extent and its padded form
+    float w_add = 0.f, y_mul = 1.f;
 };
 // act[i] <- row first + i * stride of the stream, i < count; act has ld (CONCAT: 2 ld) columns
 int residual_norm_rows(void *act, const ResidualNorm &r, int pro, int first, int stride, int count, int dtype, hipStream_t s);

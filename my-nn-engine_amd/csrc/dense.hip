@@ -35,6 +35,21 @@ int pack_blocks(const PackBlocks &p, int dtype, hipStream_t s) {
     return launch_status("pack_blocks_kernel");
 }
 
+template <typename T> __global__ void pack_taps_kernel(PackTaps p, int total) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= total) return;
+    const int j = i % p.taps, c = i / p.taps;
+    p.dst[(size_t)j * p.channels + p.ch0 + c / p.dim * p.dimp + c % p.dim] = Elem<T>::ld((const T *)p.src, i);
+}
+int pack_taps(const PackTaps &p, int dtype, hipStream_t s) {
+    const int total = p.heads * p.dim * p.taps;
+    return dispatch_dense(dtype, [&](auto *t) {
+        using T = std::remove_pointer_t<decltype(t)>;
+        MYNN_LAUNCH(pack_taps_kernel<T>, dim3((total + 255) / 256), dim3(256), 0, s, p, total);
+        return launch_status("pack_taps_kernel");
+    });
+}
+
 // ---- embedding ----------------------------------------------------------------------------------------------------------
 __device__ inline size_t history_row(const EmbedParams &p, int b, int r) { return kv_cache_row(p.paging, b, 0, r, 1, p.max_seq); }
 
@@ -101,7 +116,7 @@ __device__ inline void row_request(RowPieces<T> &q, const float *x, const T *y, 
 // act[0, ld) = x' (unnormed) or rms_norm(x') * wa; x_out (may be null) receives x'
 template <typename T>
 __device__ inline void row_finish(const RowPieces<T> &q, float *act, const float *x, const T *y, const T *wb, const T *wa, float *x_out,
-                                  float eps, int width, int ld, float *red) {
+                                  float eps, int width, int ld, float w_add, float y_mul, float *red) {
     constexpr int SPAN = kPieces * kRowThreads * 4;
     const bool one = ld <= SPAN;
     float inv_y = 0.f;
@@ -136,6 +151,8 @@ __device__ inline void row_finish(const RowPieces<T> &q, float *act, const float
                     float fy[4], fw[4];
                     yv.widen(fy);
                     wv.widen(fw);
+#pragma unroll
+                    for (int e = 0; e < 4; e++) fw[e] = (fw[e] + w_add) * y_mul;
                     v.x += fy[0] * inv_y * fw[0]; v.y += fy[1] * inv_y * fw[1];
                     v.z += fy[2] * inv_y * fw[2]; v.w += fy[3] * inv_y * fw[3];
                 }
@@ -157,7 +174,7 @@ __device__ inline void row_finish(const RowPieces<T> &q, float *act, const float
                 float fw[4];
                 wv.widen(fw);
                 float4 v = *(float4 *)(act + k);
-                v.x *= inv * fw[0]; v.y *= inv * fw[1]; v.z *= inv * fw[2]; v.w *= inv * fw[3];
+                v.x *= inv * (fw[0] + w_add); v.y *= inv * (fw[1] + w_add); v.z *= inv * (fw[2] + w_add); v.w *= inv * (fw[3] + w_add);
                 *(float4 *)(act + k) = v;
             }
         }
@@ -174,7 +191,7 @@ __global__ __launch_bounds__(kRowThreads) void residual_norm_rows_kernel(T *act_
     const T *wa = PRO == PRO_RESIDUAL_NORM ? (const T *)r.wa : nullptr;
     RowPieces<T> q;
     row_request<T>(q, x, y, (const T *)r.wb, wa, r.ld, 0);
-    row_finish<T>(q, act, x, y, (const T *)r.wb, wa, r.x_out ? r.x_out + at : nullptr, r.eps, r.width, r.ld, red);
+    row_finish<T>(q, act, x, y, (const T *)r.wb, wa, r.x_out ? r.x_out + at : nullptr, r.eps, r.width, r.ld, r.w_add, r.y_mul, red);
     T *out = act_out + (size_t)blockIdx.x * r.ld * (PRO == PRO_RESIDUAL_CONCAT ? 2 : 1);
     for (int k = threadIdx.x * 4; k < r.ld; k += kRowThreads * 4) {  // (a thread reads back what it wrote)
         store4<T>(out + k, *(const float4 *)(act + k));
@@ -206,6 +223,7 @@ int residual_norm_rows(void *act, const ResidualNorm &r, int pro, int first, int
             MYNN_LAUNCH(kernel, dim3(count), dim3(kRowThreads), lds, s, (T *)act, r, first, stride);
             return launch_status("residual_norm_rows_kernel");
         };
+        if (pro == PRO_RESIDUAL) return go(residual_norm_rows_kernel<T, PRO_RESIDUAL>);
         return pro == PRO_RESIDUAL_CONCAT ? go(residual_norm_rows_kernel<T, PRO_RESIDUAL_CONCAT>) : go(residual_norm_rows_kernel<T, PRO_RESIDUAL_NORM>);
     });
 }
@@ -280,7 +298,7 @@ __global__ __launch_bounds__(kRowThreads) void dense_gemv_kernel(const T *w, con
         RowPieces<T> q;
         row_request<T>(q, r.x, y, wb, wa, r.ld, 0);
         load(min(g, groups - 1), 0);
-        row_finish<T>(q, act, r.x, y, wb, wa, blockIdx.x == 0 ? r.x_out : nullptr, r.eps, r.width, r.ld, red);
+        row_finish<T>(q, act, r.x, y, wb, wa, blockIdx.x == 0 ? r.x_out : nullptr, r.eps, r.width, r.ld, r.w_add, r.y_mul, red);
         if constexpr (PRO == PRO_RESIDUAL_CONCAT)
             for (int k = threadIdx.x * 4; k < r.ld; k += kRowThreads * 4) *(float4 *)(act + r.ld + k) = *(const float4 *)(r.x0 + k);
     }
@@ -416,6 +434,10 @@ int dense_gemv(void *out, const void *act, const ResidualNorm *r, int pro, const
             MYNN_REQUIRE(store == DENSE_F32, MYNN_ERR_UNSUPPORTED, "dense gemv: concatenated row with store %d", store);
             return launch_gemv<T, 2, PRO_RESIDUAL_CONCAT, DENSE_F32>(out, act, rr, w, N, K, scale, s, cand, n_cand);
         }
+        if (pro == PRO_RESIDUAL) {
+            MYNN_REQUIRE(store == DENSE_F32, MYNN_ERR_UNSUPPORTED, "dense gemv: unnormed row with store %d", store);
+            return launch_gemv<T, 2, PRO_RESIDUAL, DENSE_F32>(out, act, rr, w, N, K, scale, s, cand, n_cand);
+        }
         if (pro == PRO_RESIDUAL_NORM) {
             if (store == DENSE_GEGLU) return launch_gemv<T, 4, PRO_RESIDUAL_NORM, DENSE_GEGLU>(out, act, rr, w, N, K, scale, s, cand, n_cand);
             if (store == DENSE_F32) return launch_gemv<T, 4, PRO_RESIDUAL_NORM, DENSE_F32>(out, act, rr, w, N, K, scale, s, cand, n_cand);
@@ -428,14 +450,24 @@ int dense_gemv(void *out, const void *act, const ResidualNorm *r, int pro, const
 
 // ---- many-row linear, f32: 128 x 64 outputs per workgroup, a wave owns 32 rows x 64 columns, K step 16 --------------
 typedef float f16acc_t __attribute__((ext_vector_type(16)));
-template <int STORE>
-__global__ __launch_bounds__(256) void gemm_nt_f32_kernel(float *out, const float *A, const float *B, int M, int N, int K, const float *scale) {
+// GROUPED: row tile blockIdx.y multiplies its group's weight (GroupedRows); DENSE_GEGLU then stores silu(gate) * up
+template <int STORE, bool GROUPED>
+__global__ __launch_bounds__(256) void gemm_nt_f32_kernel(float *out, const float *A, const float *B, int M, int N, int K, const float *scale, GroupedRows gr) {
     constexpr int BK = 16, LD = BK + 4;
     __shared__ __align__(16) float As[128 * LD], Bs[64 * LD];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int m0 = blockIdx.y * 128, n0 = blockIdx.x * 64;
     const int lr = tid >> 2, lc = (tid & 3) * 4;
-    const float *a0 = A + (size_t)min(m0 + lr, M - 1) * K + lc, *a1 = A + (size_t)min(m0 + lr + 64, M - 1) * K + lc;
+    if constexpr (GROUPED) {
+        const int grp = gr.tile_group[blockIdx.y];
+        if (grp < 0) return;
+        B += (size_t)grp * gr.group_elems;
+    }
+    auto a_row = [&](int r) {
+        if constexpr (GROUPED) return gr.gather ? max(gr.slot[r], 0) / gr.per_row : r;
+        else return min(r, M - 1);
+    };
+    const float *a0 = A + (size_t)a_row(m0 + lr) * K + lc, *a1 = A + (size_t)a_row(m0 + lr + 64) * K + lc;
     const float *b0 = B + (size_t)min(n0 + lr, N - 1) * K + lc;
     f16acc_t acc[2];
 #pragma unroll
@@ -463,6 +495,19 @@ __global__ __launch_bounds__(256) void gemm_nt_f32_kernel(float *out, const floa
 #pragma unroll
     for (int e = 0; e < 16; e++) {
         const int row = m0 + wave * 32 + 8 * (e >> 2) + 4 * fk + (e & 3);
+        if constexpr (GROUPED) {
+            const int as = gr.slot[row];
+            if (as < 0) continue;
+            if constexpr (STORE == DENSE_GEGLU) {
+                const float gate = acc[0][e] * gr.scale[as], up = acc[1][e] * gr.scale[as];
+                out[(size_t)row * (N / 2) + n0 / 2 + fr] = gate * sigmoidf(gate) * up;
+            } else {
+#pragma unroll
+                for (int j = 0; j < 2; j++)
+                    if (n0 + j * 32 + fr < N) out[(size_t)as * N + n0 + j * 32 + fr] = acc[j][e];
+            }
+            continue;
+        }
         if (row >= M) continue;
         if constexpr (STORE == DENSE_GEGLU) {
             out[(size_t)row * (N / 2) + n0 / 2 + fr] = gelu_tanh(acc[0][e]) * acc[1][e];
@@ -485,9 +530,24 @@ int dense_gemm(void *out, const void *act, const void *w, int M, int N, int K, i
     const dim3 grid((N + 63) / 64, (M + 127) / 128);
     MYNN_REQUIRE(grid.y <= 65535, MYNN_ERR_UNSUPPORTED, "dense gemm: M=%d", M);
     if (store == DENSE_GEGLU)
-        MYNN_LAUNCH(gemm_nt_f32_kernel<DENSE_GEGLU>, grid, dim3(256), 0, s, (float *)out, (const float *)act, (const float *)w, M, N, K, scale);
+        MYNN_LAUNCH((gemm_nt_f32_kernel<DENSE_GEGLU, false>), grid, dim3(256), 0, s, (float *)out, (const float *)act, (const float *)w, M, N, K, scale, GroupedRows{});
     else
-        MYNN_LAUNCH(gemm_nt_f32_kernel<DENSE_F32>, grid, dim3(256), 0, s, (float *)out, (const float *)act, (const float *)w, M, N, K, scale);
+        MYNN_LAUNCH((gemm_nt_f32_kernel<DENSE_F32, false>), grid, dim3(256), 0, s, (float *)out, (const float *)act, (const float *)w, M, N, K, scale, GroupedRows{});
+    return launch_status("gemm_nt_f32_kernel");
+}
+
+int gemm_grouped(void *out, const void *act, const void *wt, const GroupedRows &g, int N, int K, int epi, int dtype, hipStream_t s) {
+    MYNN_REQUIRE(out && act && wt && g.tile_group && g.slot && g.per_row > 0 && N > 0 && K > 0 && K % 64 == 0 && g.tiles > 0 && g.tiles <= 65535,
+                 MYNN_ERR_INVALID, "grouped gemm: %d tiles, N=%d K=%d", g.tiles, N, K);
+    MYNN_REQUIRE(g.gather == (epi == GEMM_SILU) && (epi != GEMM_SILU || (N % 64 == 0 && g.scale)), MYNN_ERR_INVALID, "grouped gemm: store %d of N=%d", epi, N);
+    if (dtype == MYNN_BF16) return gemm_grouped_bf16(out, act, wt, g, N, K, epi, s);
+    MYNN_REQUIRE(dtype == MYNN_F32, MYNN_ERR_UNSUPPORTED, "grouped gemm: dtype %d", dtype);
+    static_assert(kGroupRows == 128, "the f32 kernel's row tile");
+    const dim3 grid((N + 63) / 64, g.tiles);
+    if (epi == GEMM_SILU)
+        MYNN_LAUNCH((gemm_nt_f32_kernel<DENSE_GEGLU, true>), grid, dim3(256), 0, s, (float *)out, (const float *)act, (const float *)wt, 0, N, K, nullptr, g);
+    else
+        MYNN_LAUNCH((gemm_nt_f32_kernel<DENSE_F32, true>), grid, dim3(256), 0, s, (float *)out, (const float *)act, (const float *)wt, 0, N, K, nullptr, g);
     return launch_status("gemm_nt_f32_kernel");
 }
 

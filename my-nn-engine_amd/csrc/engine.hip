@@ -1,7 +1,8 @@
 // One checkpoint on the device and the sessions it serves: config.json through the model registry, weights uploaded once,
 // one weight set, and per session a decode executor and a prompt executor over a cache of its own.  Layered models (and
 // Llama shapes that have a paged form) take their cache rows from one pool of pages, so sessions of different lengths share
-// the memory and a session that ends gives its pages to the next.  Host code; the executors do the rest.
+// the memory and a session that ends gives its pages to the next; its sequence states go to the next session the same way.
+// Host code; the executors do the rest.
 #include <algorithm>
 #include <memory>
 #include <vector>
@@ -20,6 +21,7 @@ struct mynn_engine {
     mynn_weight_set *set = nullptr;
     mynn_kv_pool *pool = nullptr;      // null: a session owns contiguous caches
     std::vector<void *> pool_buffers;
+    std::vector<std::vector<void *>> slots;  // sequence states of ended sessions (one buffer per state), for the next ones
     int sessions = 0;
     int prefill_rows = 0;
 };
@@ -28,17 +30,20 @@ namespace {
 struct EngineSession {
     mynn_engine *engine;
     mynn_kv_pages *pages = nullptr;
-    std::vector<void *> caches;
+    std::vector<void *> caches;  // contiguous caches (no pool)
+    std::vector<void *> slot;    // sequence states
 };
 
-int state_buffers(const mynn_engine &e, size_t rows, std::vector<void *> &out) {
+// the session-state buffers with a row per token (PER_TOKEN) or a block per sequence; null where the other kind belongs
+enum StateKind { PER_TOKEN, PER_SEQUENCE };
+int state_buffers(const mynn_engine &e, StateKind kind, size_t rows, std::vector<void *> &out) {
     const int n = mynn_arch_state_count(e.arch);
     for (int i = 0; i < n; i++) {
         void *p = nullptr;
-        const size_t bytes = rows * mynn_arch_state_row_bytes(e.arch, i, e.opt.dtype);
-        MYNN_HIP(hipMalloc(&p, bytes));
+        const size_t bytes = kind == PER_TOKEN ? rows * mynn_arch_state_row_bytes(e.arch, i, e.opt.dtype) : mynn_arch_state_seq_bytes(e.arch, i);
+        if (bytes) MYNN_HIP(hipMalloc(&p, bytes));
         out.push_back(p);
-        MYNN_HIP(hipMemset(p, 0, bytes));
+        if (bytes) MYNN_HIP(hipMemset(p, 0, bytes));
     }
     return 0;
 }
@@ -71,7 +76,7 @@ int open_engine(mynn_engine &e, const char *dir, const mynn_engine_options &opt)
         const int n_pages = (e.opt.max_tokens + P - 1) / P + 8;  // (a session's last page is rarely full)
         e.pool = mynn_kv_pool_create(n_pages, P);
         if (!e.pool) return MYNN_ERR_INVALID;
-        rc = state_buffers(e, (size_t)n_pages * P, e.pool_buffers);
+        rc = state_buffers(e, PER_TOKEN, (size_t)n_pages * P, e.pool_buffers);
     }
     return rc;
 }
@@ -82,6 +87,7 @@ void release_session(mynn_llm *l) {
     if (l->decode) model_destroy(l->decode);
     if (s->pages) (void)mynn_kv_pages_destroy(s->pages);
     for (void *p : s->caches) (void)hipFree(p);
+    if (!s->slot.empty()) s->engine->slots.push_back(std::move(s->slot));
     s->engine->sessions--;
     delete s;
 }
@@ -94,6 +100,8 @@ extern "C" int mynn_engine_close(mynn_engine *e) {
     if (e->weights) mynn_device_weights_free(e->weights);
     if (e->pool) (void)mynn_kv_pool_destroy(e->pool);
     for (void *p : e->pool_buffers) (void)hipFree(p);
+    for (auto &slot : e->slots)
+        for (void *p : slot) (void)hipFree(p);
     delete e;
     return 0;
 }
@@ -128,13 +136,21 @@ extern "C" mynn_llm *mynn_engine_session(mynn_engine *e, int64_t eos_token_id) {
     e->sessions++;
     std::vector<void *> state = e->pool_buffers;
     bool ok = true;
-    if (e->pool) {
+    if (e->slots.empty()) ok = state_buffers(*e, PER_SEQUENCE, 1, s->slot) == 0;
+    else {
+        s->slot = std::move(e->slots.back());
+        e->slots.pop_back();
+    }
+    if (ok && !e->pool) {
+        ok = state_buffers(*e, PER_TOKEN, e->opt.max_seq, s->caches) == 0;
+        state = s->caches;
+    }
+    for (size_t i = 0; ok && i < state.size(); i++)
+        if (s->slot[i]) state[i] = s->slot[i];
+    if (ok && e->pool) {
         s->pages = mynn_kv_pages_create(e->pool, 1, e->opt.max_seq);
         ok = s->pages != nullptr;
         state.push_back(s->pages);
-    } else {
-        ok = state_buffers(*e, e->opt.max_seq, s->caches) == 0;
-        state = s->caches;
     }
     mynn_model_config cfg = e->cfg;
     if (ok) l->decode = mynn_model_create_shared(&cfg, e->set, state.data());
@@ -147,5 +163,6 @@ extern "C" mynn_llm *mynn_engine_session(mynn_engine *e, int64_t eos_token_id) {
     l->prefill_len = l->prefill ? cfg.seq_q : 0;
     l->max_seq = e->opt.max_seq;
     l->eos = eos_token_id;
+    l->seq_state = model_has_sequence_state(l->decode);
     return l;
 }

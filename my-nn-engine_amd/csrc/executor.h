@@ -175,6 +175,10 @@ void destroy_layered(Model &m);
 // ---- decoder.hip: a model that takes any number of new tokens up to seq_q in a step (a Llama graph of seq_q > 1 takes
 // exactly seq_q; shorter portions are padded and their last rows written over by the next tokens)
 bool model_takes_any_rows(const void *state);
+// ---- layered.hip: models whose session state stands for all tokens read so far; a copy of it and back (on the model's stream)
+bool model_has_sequence_state(const void *state);
+int executor_save_state(void *state);
+int executor_restore_state(void *state);
 int executor_bind_pages(Model &m);
 
 }  // namespace mynn

@@ -101,7 +101,7 @@ __device__ __forceinline__ void gemm_store(AccAt at, uint16_t *lds, T *C, const 
                                            int n0, int wrow, int wcol, int lane, int wave) {
     constexpr int TI = G::TI, TJ = G::TJ;
     constexpr int EST = G::EST;
-    constexpr bool GATED = EPI == GEMM_SWIGLU || EPI == GEMM_GEGLU;
+    constexpr bool GATED = EPI == GEMM_SWIGLU || EPI == GEMM_GEGLU || EPI == GEMM_SILU;
     static_assert(!GATED || TJ % 2 == 0, "the gated stores pair neighbouring column tiles");
     if constexpr (EPI == GEMM_F32) {
         // f32 straight from the accumulators: four neighbouring columns of a row per lane
@@ -139,7 +139,7 @@ __device__ __forceinline__ void gemm_store(AccAt at, uint16_t *lds, T *C, const 
         T *prow = patch + (lane & 31) * EST + (lane >> 5) * 4;
 #pragma unroll
         for (int q = 0; q < 4; q++) {
-            if constexpr (EPI == GEMM_GEGLU) {
+            if constexpr (EPI == GEMM_GEGLU || EPI == GEMM_SILU) {
                 // (gate and up enter the activation as the f32 sums they are)
 #pragma unroll
                 for (int j = 0; j < TJ; j += 2) {
@@ -147,7 +147,8 @@ __device__ __forceinline__ void gemm_store(AccAt at, uint16_t *lds, T *C, const 
 #pragma unroll
                     for (int x = 0; x < 4; x++) {
                         const float g = at(i, j, 4 * q + x), u = at(i, j + 1, 4 * q + x);
-                        o[x] = g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(gelu_tanh_arg(g) * -1.4426950408889634f)) * u;
+                        const float z = EPI == GEMM_SILU ? g : gelu_tanh_arg(g);
+                        o[x] = g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.4426950408889634f)) * u;
                     }
                     *(uint2 *)(prow + j * 16 + 8 * q) = uint2{pack2<T>(o[0], o[1]), pack2<T>(o[2], o[3])};
                 }
@@ -315,10 +316,10 @@ template <typename G> constexpr size_t dma_lds_bytes() { return (size_t)2 * dma_
 typedef int i4x_t __attribute__((ext_vector_type(4)));
 typedef int i16x_t __attribute__((ext_vector_type(16)));
 
-template <typename T, typename G, int EPI, bool I8>
-__global__ __launch_bounds__(G::THREADS) void gemm_nt_dma_kernel(T *C, const void *A_, const void *B_, const T *R, int M, int N,
-                                                                 int K, int Kp, const T *a_scale, const T *b_scale,
-                                                                 int32_t *acc_out) {
+// GROUPED: row tile tm multiplies its group's weight, rows come from and go to where GroupedRows says.
+template <typename T, typename G, int EPI, bool I8, bool GROUPED>
+__device__ __forceinline__ void gemm_dma_body(T *C, const void *A_, const void *B_, const T *R, int M, int N, int K, int Kp, const T *a_scale,
+                                              const T *b_scale, int32_t *acc_out, const GroupedRows &gr) {
     constexpr int TI = G::TI, TJ = G::TJ, KS = DBK / 16, BM = G::BM, BN = G::BN;
     constexpr int EB = I8 ? 1 : 2;            // bytes per operand value
     constexpr int TILE_B = DBK * 2;           // bytes of one row of a K tile
@@ -334,13 +335,23 @@ __global__ __launch_bounds__(G::THREADS) void gemm_nt_dma_kernel(T *C, const voi
     int tm, tn;
     tile_of(blockIdx.x, gridDim.x, tiles_m, tiles_n, tm, tn);
     const int m0 = tm * BM, n0 = tn * BN;
+    if constexpr (GROUPED) {
+        static_assert(BM == kGroupRows, "a row tile is one group's");
+        const int grp = gr.tile_group[tm];
+        if (grp < 0) return;
+        B += (size_t)grp * gr.group_elems * EB;
+    }
+    auto a_row = [&](int r) {
+        if constexpr (GROUPED) return EPI == GEMM_SILU ? max(gr.slot[r], 0) / gr.per_row : r;
+        else return min(r, M - 1);
+    };
 
     // this lane's chunks of each operand tile: LDS position P = (CH*wave + i)*64 + lane
     const char *asrc[CHA], *bsrc[CHB];
 #pragma unroll
     for (int i = 0; i < CHA; i++) {
         const int P = (CHA * wave + i) * 64 + lane, r = P >> 3, c = (P & 7) ^ ((r >> 1) & 7);
-        asrc[i] = A + (size_t)min(m0 + r, M - 1) * K * EB + c * 16;
+        asrc[i] = A + (size_t)a_row(m0 + r) * K * EB + c * 16;
     }
 #pragma unroll
     for (int i = 0; i < CHB; i++) {
@@ -492,10 +503,48 @@ __global__ __launch_bounds__(G::THREADS) void gemm_nt_dma_kernel(T *C, const voi
             gemm_store<T, G, EPI>([&](int i, int j, int e) { return ((float)acc[i][j][e] * asc[i]) * bw[j * 32 + 8 * (e >> 2) + (e & 3)]; },
                                   lds, C, R, M, N, m0, n0, wrow, wcol, lane, wave);
         }
+    } else if constexpr (GROUPED && EPI == GEMM_SILU) {
+        float rs[TI];
+#pragma unroll
+        for (int i = 0; i < TI; i++) {
+            const int as = gr.slot[m0 + wrow + i * 32 + (lane & 31)];
+            rs[i] = as < 0 ? 0.f : gr.scale[as];
+        }
+        gemm_store<T, G, EPI>([&](int i, int j, int e) { return acc[i][j][e] * rs[i]; }, lds, C, R, M, N, m0, n0, wrow, wcol, lane, wave);
+    } else if constexpr (GROUPED) {
+        // rows scattered to their assignments: four neighbouring columns of a row per lane
+#pragma unroll
+        for (int i = 0; i < TI; i++) {
+            const int as = gr.slot[m0 + wrow + i * 32 + (lane & 31)];
+            if (as < 0) continue;
+#pragma unroll
+            for (int j = 0; j < TJ; j++)
+#pragma unroll
+                for (int q = 0; q < 4; q++) {
+                    const int col = n0 + wcol + j * 32 + 8 * q + 4 * (lane >> 5);
+                    if (col + 4 > N) continue;  // (N % 4 == 0)
+                    const float4 v = float4{acc[i][j][4 * q], acc[i][j][4 * q + 1], acc[i][j][4 * q + 2], acc[i][j][4 * q + 3]};
+                    if constexpr (EPI == GEMM_F32) *(float4 *)((float *)C + (size_t)as * N + col) = v;
+                    else *(uint2 *)(C + (size_t)as * N + col) = uint2{pack2<T>(v.x, v.y), pack2<T>(v.z, v.w)};
+                }
+        }
     } else {
         gemm_store<T, G, EPI>([&](int i, int j, int e) { return acc[i][j][e]; }, lds, C, R, M, N, m0, n0, wrow, wcol, lane, wave);
     }
 }
+
+template <typename T, typename G, int EPI, bool I8>
+__global__ __launch_bounds__(G::THREADS) void gemm_nt_dma_kernel(T *C, const void *A_, const void *B_, const T *R, int M, int N,
+                                                                 int K, int Kp, const T *a_scale, const T *b_scale,
+                                                                 int32_t *acc_out) {
+    gemm_dma_body<T, G, EPI, I8, false>(C, A_, B_, R, M, N, K, Kp, a_scale, b_scale, acc_out, GroupedRows{});
+}
+using TileGroup = GemmTile<kGroupRows, 256, 2, 4>;  // 64 x 64 per wave
+template <typename T, typename G, int EPI>
+__global__ __launch_bounds__(G::THREADS) void gemm_nt_grouped_kernel(T *C, const void *A, const void *B, int N, int K, GroupedRows gr) {
+    gemm_dma_body<T, G, EPI, false, true>(C, A, B, nullptr, gr.tiles * G::BM, N, K, K, nullptr, nullptr, nullptr, gr);
+}
+
 
 static int gemm_kp(int K) { return (K + 2 * BK - 1) / (2 * BK) * (2 * BK); }  // the GEMM walks K in pairs of steps
 
@@ -553,6 +602,20 @@ static int gemm_launch_dma(void *out, const void *act, const void *wt, const voi
     MYNN_LAUNCH((gemm_nt_dma_kernel<T, G, EPI, I8>), dim3(tiles), dim3(G::THREADS), dma_lds_bytes<G>(), s, (T *)out, act, wt,
                 (const T *)res, M, N, K, I8 ? K : gemm_kp(K), (const T *)a_scale, (const T *)b_scale, acc_out);
     return launch_status("gemm_nt_dma_kernel");
+}
+
+int gemm_grouped_bf16(void *out, const void *act, const void *wt, const GroupedRows &g, int N, int K, int epi, hipStream_t s) {
+    MYNN_REQUIRE(K % 64 == 0 && N % 4 == 0 && aligned16(act) && aligned16(wt), MYNN_ERR_INVALID, "grouped gemm: N=%d K=%d", N, K);
+    auto go = [&](auto kernel) {
+        constexpr size_t lds = dma_lds_bytes<TileGroup>();
+        MYNN_HIP(hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+        MYNN_LAUNCH(kernel, dim3(g.tiles * ((N + TileGroup::BN - 1) / TileGroup::BN)), dim3(TileGroup::THREADS), lds, s, (bf16_t *)out, act, wt, N, K, g);
+        return launch_status("gemm_nt_grouped_kernel");
+    };
+    if (epi == GEMM_SILU) return go(gemm_nt_grouped_kernel<bf16_t, TileGroup, GEMM_SILU>);
+    if (epi == GEMM_F32) return go(gemm_nt_grouped_kernel<bf16_t, TileGroup, GEMM_F32>);
+    MYNN_REQUIRE(epi == GEMM_PLAIN, MYNN_ERR_UNSUPPORTED, "grouped gemm: store %d", epi);
+    return go(gemm_nt_grouped_kernel<bf16_t, TileGroup, GEMM_PLAIN>);
 }
 
 // QuantizedMatMul on the matrix cores for a grid of at least one round of 256-row tiles: K % 128 == 0.

@@ -1,11 +1,13 @@
-// Executor of decoders described layer by layer (ModelSpec): a 32-bit residual stream, sandwich-normed layers whose mixer
-// and feed-forward come from the description, and layer ranges that run several times.  It fills the executor's build and
+// Executor of decoders described layer by layer (ModelSpec): a 32-bit residual stream, layers with norms behind (and, if the
+// description says so, in front of) their sublayers, whose mixer and feed-forward come from the description, and layer ranges
+// that run several times.  It fills the executor's build and
 // enqueue hooks; inputs, pages, graph capture, the device-resident loop, profile and session are decoder.hip's and
 // llm_session.hip's, the same as for the Llama graph.
 //
-// Session state: a cache per layer run (a looped layer has one per pass), [batch, max_seq, row] or pages of it, then the
-// token history [batch, max_seq] int32 in the same rows: a pair embedding reads a step's previous token there, so it is
-// found again after a rewind, in any portion and on any page.
+// Session state: a cache per layer run with attention (a looped layer has one per pass), [batch, max_seq, row] or pages of it,
+// then the token history [batch, max_seq] int32 in the same rows: a pair embedding reads a step's previous token there, so it
+// is found again after a rewind, in any portion and on any page.  Runs with a recurrence or a short convolution have a block
+// per sequence behind these, which a step from position 0 starts afresh.
 //
 // One new token (decode, batch 1): per run the input projection [norms and residual sum in its prologue], latent_prepare,
 // attention, merge + W_uv + gate, output projection, gate/up, down -- 7 launches; all scalars in device memory, captured
@@ -13,27 +15,10 @@
 #include <algorithm>
 #include <cmath>
 
-#include "executor.h"
-#include "latent_attention.h"
+#include "layered.h"
 
 namespace mynn {
 
-// a linear's rows in the storage type, padded [N, K]
-struct DenseW {
-    void *w = nullptr;
-    int N = 0, K = 0;
-};
-struct LayerWeights {
-    void *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr, *latent_norm = nullptr;
-    DenseW in, ukv, o, gu, down;
-};
-struct LayeredWeights {
-    std::vector<LayerWeights> layers;
-    DenseW loop_in, head;
-    void *final_norm = nullptr;
-    std::vector<void *> owned;
-    bool ready = false;
-};
 void layered_weights_free(LayeredWeights *w) {
     if (!w) return;
     for (void *p : w->owned) (void)hipFree(p);
@@ -44,29 +29,56 @@ void layered_weights_free(LayeredWeights *w) {
 // expanded form's with the number of keys it has to expand)
 constexpr int kAbsorbRows = 32;
 
-struct LayeredNet {
-    std::shared_ptr<const ModelSpec> spec;
-    const LayeredWeights *w = nullptr;
-    const void *embed = nullptr, *bigram = nullptr;  // the caller's tables
-    std::vector<void *> caches;   // per run
-    int32_t *history = nullptr;
-    std::vector<float2 *> rot;    // per layer, into rot_tables
-    std::vector<void *> rot_tables;
-    int ld = 0;                   // padded width
-    float *xa = nullptr, *xb = nullptr, *x0 = nullptr, *logit_scale = nullptr;
-    void *act = nullptr, *proj = nullptr, *attn = nullptr, *y = nullptr, *hmid = nullptr, *q_abs = nullptr;
-    void *c_rows = nullptr, *rot_rows = nullptr, *kv = nullptr;
-    float *part_o = nullptr, *part_ml = nullptr;
-    GreedyCand *cand = nullptr;
-    bool gemv = false;            // every linear fits the one-row kernel
-};
 void destroy_layered(Model &m) {
     for (void *p : m.net->rot_tables) (void)hipFree(p);
+    if (m.net->saved) (void)hipFree(m.net->saved);
     delete m.net;
     m.net = nullptr;
 }
 
 // ---- padded weight copies, once per weight set ------------------------------------------------------------------------
+int WeightPacker::alloc(void **p, size_t rows, size_t cols, size_t elem) {
+    const size_t bytes = rows * cols * (elem ? elem : dtype_size(dt));
+    MYNN_HIP(hipMalloc(p, bytes));
+    w.owned.push_back(*p);
+    m.wset->bytes_repack += bytes;
+    MYNN_HIP(hipMemsetAsync(*p, 0, bytes, m.stream));
+    return 0;
+}
+int WeightPacker::vec(void **p, const std::string &name, int heads, int n, int np, int padded) {
+    TRY(alloc(p, 1, padded));
+    return pack_blocks(PackBlocks{*p, src(name), padded, (long)heads * n, 1, 1, 0, 1, 0, 1, heads, n, 0, np, n, 0, 0}, dt, m.stream);
+}
+int WeightPacker::rows(DenseW &l, const std::string &name, int heads, int n, int np, int row0) {
+    return pack_blocks(PackBlocks{l.w, src(name), l.K, s.width, heads, n, row0, np, 0, n, 1, s.width, 0, s.width, s.width, 0, 0}, dt, m.stream);
+}
+int WeightPacker::cols(DenseW &l, const std::string &name, int heads, int n, int np, int col0) {
+    return pack_blocks(PackBlocks{l.w, src(name), l.K, (long)heads * n, 1, s.width, 0, s.width, 0, s.width, heads, n, col0, np, n, 0, 0}, dt, m.stream);
+}
+
+static int pack_latent(WeightPacker &pk, LayerWeights &o, const MixerSpec &mix, const std::string &mx) {
+    const int W = pk.s.width, ld = pk.ld;
+    const LatentDims d = latent_dims(mix);
+    TRY(pk.norm(&o.latent_norm, mx + "dkv.norm", d.rank, d.rp));
+    // input projection: q head by head [dim | rotated], latent, rotated key part, gates
+    TRY(pk.linear(o.in, d.n_in(), ld));
+    auto in_rows = [&](const char *t, int H, int rows, int dst0, int dst_rs, int src0, int src_rs) {
+        return pack_blocks(PackBlocks{o.in.w, pk.src(mx + t), ld, W, H, rows, dst0, dst_rs, src0, src_rs, 1, W, 0, W, W, 0, 0}, pk.dt, pk.m.stream);
+    };
+    TRY(in_rows("q", d.H, d.dim, 0, d.dk(), 0, d.dim + d.rot));
+    TRY(in_rows("q", d.H, d.rot, d.dimp, d.dk(), d.dim, d.dim + d.rot));
+    TRY(in_rows("dkv", 1, d.rank, d.qcols(), 1, 0, 1));
+    TRY(in_rows("dkv", 1, d.rot, d.qcols() + d.rp, 1, d.rank, 1));
+    TRY(in_rows("g", 1, d.H, d.qcols() + d.lw(), 1, 0, 1));
+    // key rows of every head, then value rows
+    TRY(pk.linear(o.ukv, d.kvcols(), d.rp));
+    TRY(pack_blocks(PackBlocks{o.ukv.w, pk.src(mx + "uk"), d.rp, d.rank, d.H, d.dim, 0, d.dimp, 0, d.dim, 1, d.rank, 0, d.rank, d.rank, 0, 0}, pk.dt, pk.m.stream));
+    TRY(pack_blocks(PackBlocks{o.ukv.w, pk.src(mx + "uv"), d.rp, d.rank, d.H, d.vdim, d.H * d.dimp, d.vdimp, 0, d.vdim, 1, d.rank, 0, d.rank, d.rank, 0, 0}, pk.dt, pk.m.stream));
+    TRY(pk.linear(o.o, ld, d.acols()));
+    TRY(pack_blocks(PackBlocks{o.o.w, pk.src(mx + "o"), d.acols(), (long)d.H * d.vdim, 1, W, 0, W, 0, W, d.H, d.vdim, 0, d.vdimp, d.vdim, 0, 0}, pk.dt, pk.m.stream));
+    return 0;
+}
+
 static int make_weights(Model &m, const ModelSpec &s) {
     WeightSet &ws = *m.wset;
     if (ws.layered && ws.layered->ready) return 0;
@@ -74,58 +86,29 @@ static int make_weights(Model &m, const ModelSpec &s) {
     ws.layered = new LayeredWeights;
     LayeredWeights &w = *ws.layered;
     const int dt = m.cfg.dtype, W = s.width, ld = pad_to(W, 64);
-    const size_t eb = dtype_size(dt);
     ws.bytes_repack = 0;
-    auto alloc = [&](void **p, size_t rows, size_t cols) {
-        MYNN_HIP(hipMalloc(p, rows * cols * eb));
-        w.owned.push_back(*p);
-        ws.bytes_repack += rows * cols * eb;
-        MYNN_HIP(hipMemsetAsync(*p, 0, rows * cols * eb, m.stream));
-        return 0;
-    };
-    auto src = [&](const std::string &name) -> const void * {
-        const int i = s.tensor_index(name);
-        return i < 0 ? nullptr : ws.initializer[i];
-    };
+    WeightPacker pk{m, w, s, dt, ld};
     for (size_t i = 0; i < s.tensors.size(); i++)
         MYNN_REQUIRE(ws.initializer[i], MYNN_ERR_INVALID, "model_init: null weight %s", s.tensors[i].name.c_str());
-    auto norm = [&](void **p, const std::string &name, int n, int padded) {
-        TRY(alloc(p, 1, padded));
-        return pack_blocks(PackBlocks{*p, src(name), padded, n, 1, 1, 0, 1, 0, 1, 1, n, 0, n, n, 0, 0}, dt, m.stream);
-    };
-    auto linear = [&](DenseW &l, int N, int K) {
-        l.N = N;
-        l.K = K;
-        return alloc(&l.w, N, K);
-    };
+    auto src = [&](const std::string &name) { return pk.src(name); };
+    auto norm = [&](void **p, const std::string &name, int n, int padded) { return pk.norm(p, name, n, padded); };
+    auto linear = [&](DenseW &l, int N, int K) { return pk.linear(l, N, K); };
     w.layers.resize(s.layers.size());
     for (size_t i = 0; i < s.layers.size(); i++) {
         const LayerSpec &L = s.layers[i];
         const std::string p = "l" + std::to_string(i) + ".", mx = p + "mix.";
         LayerWeights &o = w.layers[i];
-        TRY(norm(&o.norm1, p + "norm1", W, ld));
-        TRY(norm(&o.norm1b, p + "norm1b", W, ld));
-        const LatentDims d = latent_dims(L.mixer);
-        TRY(norm(&o.latent_norm, mx + "dkv.norm", d.rank, d.rp));
-        // input projection: q head by head [dim | rotated], latent, rotated key part, gates
-        TRY(linear(o.in, d.n_in(), ld));
-        auto in_rows = [&](const char *t, int H, int rows, int dst0, int dst_rs, int src0, int src_rs) {
-            return pack_blocks(PackBlocks{o.in.w, src(mx + t), ld, W, H, rows, dst0, dst_rs, src0, src_rs, 1, W, 0, W, W, 0, 0}, dt, m.stream);
-        };
-        TRY(in_rows("q", d.H, d.dim, 0, d.dk(), 0, d.dim + d.rot));
-        TRY(in_rows("q", d.H, d.rot, d.dimp, d.dk(), d.dim, d.dim + d.rot));
-        TRY(in_rows("dkv", 1, d.rank, d.qcols(), 1, 0, 1));
-        TRY(in_rows("dkv", 1, d.rot, d.qcols() + d.rp, 1, d.rank, 1));
-        TRY(in_rows("g", 1, d.H, d.qcols() + d.lw(), 1, 0, 1));
-        // key rows of every head, then value rows
-        TRY(linear(o.ukv, d.kvcols(), d.rp));
-        TRY(pack_blocks(PackBlocks{o.ukv.w, src(mx + "uk"), d.rp, d.rank, d.H, d.dim, 0, d.dimp, 0, d.dim, 1, d.rank, 0, d.rank, d.rank, 0, 0}, dt, m.stream));
-        TRY(pack_blocks(PackBlocks{o.ukv.w, src(mx + "uv"), d.rp, d.rank, d.H, d.vdim, d.H * d.dimp, d.vdimp, 0, d.vdim, 1, d.rank, 0, d.rank, d.rank, 0, 0}, dt, m.stream));
-        TRY(linear(o.o, ld, d.acols()));
-        TRY(pack_blocks(PackBlocks{o.o.w, src(mx + "o"), d.acols(), (long)d.H * d.vdim, 1, W, 0, W, 0, W, d.H, d.vdim, 0, d.vdimp, d.vdim, 0, 0}, dt, m.stream));
-        if (L.mlp.kind == MlpSpec::NONE) continue;
-        TRY(norm(&o.norm2, p + "norm2", W, ld));
-        TRY(norm(&o.norm2b, p + "norm2b", W, ld));
+        if (s.pre_norm) TRY(norm(&o.norm1, p + "norm1", W, ld));
+        TRY(norm(&o.norm1b, p + (s.pre_norm ? "norm1b" : "norm1"), W, ld));
+        if (L.mlp.kind != MlpSpec::NONE) {
+            if (s.pre_norm) TRY(norm(&o.norm2, p + "norm2", W, ld));
+            TRY(norm(&o.norm2b, p + (s.pre_norm ? "norm2b" : "norm2"), W, ld));
+        }
+        if (L.mlp.kind == MlpSpec::EXPERTS) TRY(pack_experts(pk, o, L.mlp, p + "mlp."));
+        if (L.mixer.kind == MixerSpec::PARALLEL) TRY(pack_parallel(pk, o, L.mixer, mx));
+        if (L.mixer.kind == MixerSpec::CHANNEL_DELTA) TRY(pack_channel_delta(pk, o, L.mixer, mx));
+        if (L.mixer.kind == MixerSpec::LATENT_ATTENTION) TRY(pack_latent(pk, o, L.mixer, mx));
+        if (L.mlp.kind != MlpSpec::GATED_DENSE) continue;
         const int F = L.mlp.ff, Fp = pad_to(F, 64);
         TRY(linear(o.gu, 2 * Fp, ld));
         TRY(pack_blocks(PackBlocks{o.gu.w, src(p + "mlp.gate"), ld, W, 1, F, 0, F, 0, F, 1, W, 0, W, W, 32, 0}, dt, m.stream));
@@ -145,19 +128,24 @@ static int make_weights(Model &m, const ModelSpec &s) {
     return 0;
 }
 
-// (cos, sin) of every position, angles in double, one table per distinct (base, dims)
+// (cos, sin) of every position, angles in double, one table per distinct rotation
 static int make_rotary_tables(LayeredNet &n, int max_seq) {
     const ModelSpec &s = *n.spec;
     n.rot.assign(s.layers.size(), nullptr);
+    auto rotary = [&](size_t i) -> const RotarySpec & {
+        const MixerSpec &m = s.layers[i].mixer;
+        return m.kind == MixerSpec::PARALLEL ? m.window.rot : m.rot;
+    };
     for (size_t i = 0; i < s.layers.size(); i++) {
-        const RotarySpec &r = s.layers[i].mixer.rot;
+        const RotarySpec &r = rotary(i);
+        if (!r.dims) continue;
         for (size_t j = 0; j < i && !n.rot[i]; j++)
-            if (s.layers[j].mixer.rot.base == r.base && s.layers[j].mixer.rot.dims == r.dims) n.rot[i] = n.rot[j];
+            if (rotary(j) == r) n.rot[i] = n.rot[j];
         if (n.rot[i]) continue;
         const int half = r.dims / 2;
         std::vector<float2> t((size_t)max_seq * half);
         for (int k = 0; k < half; k++) {
-            const double f = pow(r.base, -2.0 * k / r.dims);
+            const double f = r.frequency(k);
             for (int p = 0; p < max_seq; p++) t[(size_t)p * half + k] = float2{(float)cos(p * f), (float)sin(p * f)};
         }
         void *d = nullptr;
@@ -184,50 +172,74 @@ int build_layered(Model &m, void **state) {
         if (s.bigram.buckets) n.bigram = m.wset->initializer[s.tensor_index("bigram")];
     }
     TRY(make_rotary_tables(n, c.max_seq));
-    n.caches.assign(state, state + s.runs.size());
-    n.history = (int32_t *)state[s.runs.size()];
-    for (void *p : n.caches) MYNN_REQUIRE(p && aligned16(p), MYNN_ERR_INVALID, "model_init: null or misaligned cache buffer");
-    MYNN_REQUIRE(n.history, MYNN_ERR_INVALID, "model_init: null token history buffer");
+    for (size_t i = 0; i < s.states.size(); i++)
+        MYNN_REQUIRE(state[i] && ((int)i == s.history || aligned16(state[i])), MYNN_ERR_INVALID, "model_init: null or misaligned state buffer %zu", i);
+    for (const LayerRun &r : s.runs) {
+        n.caches.push_back(r.cache < 0 ? nullptr : state[r.cache]);
+        n.memory.push_back(r.memory < 0 ? nullptr : (float *)state[r.memory]);
+    }
+    n.history = (int32_t *)state[s.history];
     if (c.kv_page_rows) {
-        m.pages = (mynn_kv_pages *)state[s.runs.size() + 1];
+        m.pages = (mynn_kv_pages *)state[s.states.size()];
         TRY(executor_bind_pages(m));
     }
 
     const int rows = c.batch * c.seq_q, ld = n.ld = pad_to(s.width, 64);
     const size_t eb = dtype_size(c.dtype);
     const int abs_rows = std::min(c.seq_q, kAbsorbRows);
-    size_t n_in = 0, acols = 0, fp = 0, q_abs = 0, part_o = 0, part_ml = 0, c_rows = 0, rot_rows = 0, kv = 0;
+    MixerScratch sc;
+    size_t q_abs = 0, c_rows = 0, rot_rows = 0, kv = 0;
     n.gemv = dense_gemv_supported(ld) && (!s.loop.times || dense_gemv_supported(2 * ld));
     for (const LayerSpec &L : s.layers) {
-        const LatentDims d = latent_dims(L.mixer);
-        n_in = std::max<size_t>(n_in, d.n_in());
-        acols = std::max<size_t>(acols, d.acols());
-        fp = std::max<size_t>(fp, L.mlp.kind == MlpSpec::NONE ? 0 : pad_to(L.mlp.ff, 64));
-        const bool expanded = latent_expanded_supported(d, c.dtype);
-        const size_t absorbed = (size_t)c.batch * (expanded ? abs_rows : c.seq_q);
-        size_t parts = 0;  // (row, head) x ranges of any portion
-        for (int S = 1; S <= (expanded ? abs_rows : c.seq_q); S++)
-            parts = std::max(parts, (size_t)c.batch * S * d.H * latent_absorbed_splits(c.batch, S, d, c.max_seq, c.dtype));
-        q_abs = std::max(q_abs, absorbed * d.H * d.lw());
-        part_o = std::max(part_o, parts * d.rp);
-        part_ml = std::max(part_ml, parts * 2);
-        if (expanded && c.seq_q > kAbsorbRows) {
-            c_rows = std::max(c_rows, (size_t)c.max_seq * d.rp);
-            rot_rows = std::max(rot_rows, (size_t)c.max_seq * d.rotp);
-            kv = std::max(kv, (size_t)c.max_seq * d.kvcols());
+        TRY(check_mixer(L.mixer));
+        int acols = 0;
+        if (L.mixer.kind == MixerSpec::LATENT_ATTENTION) {
+            const LatentDims d = latent_dims(L.mixer);
+            sc.proj = std::max<size_t>(sc.proj, (size_t)rows * d.n_in() * eb);
+            acols = d.acols();
+            const bool expanded = latent_expanded_supported(d, c.dtype);
+            const size_t absorbed = (size_t)c.batch * (expanded ? abs_rows : c.seq_q);
+            size_t parts = 0;  // (row, head) x ranges of any portion
+            for (int S = 1; S <= (expanded ? abs_rows : c.seq_q); S++)
+                parts = std::max(parts, (size_t)c.batch * S * d.H * latent_absorbed_splits(c.batch, S, d, c.max_seq, c.dtype));
+            q_abs = std::max(q_abs, absorbed * d.H * d.lw());
+            sc.part_o = std::max(sc.part_o, parts * d.rp * 4);
+            sc.part_ml = std::max(sc.part_ml, parts * 2 * 4);
+            if (expanded && c.seq_q > kAbsorbRows) {
+                c_rows = std::max(c_rows, (size_t)c.max_seq * d.rp);
+                rot_rows = std::max(rot_rows, (size_t)c.max_seq * d.rotp);
+                kv = std::max(kv, (size_t)c.max_seq * d.kvcols());
+            }
+        } else {
+            scratch_recurrent(sc, L.mixer, c);
+            acols = L.mixer.kind == MixerSpec::PARALLEL ? parallel_dims(L.mixer).acols() : delta_dims(L.mixer.delta).acols();
         }
-        n.gemv = n.gemv && dense_gemv_supported(d.acols()) && (L.mlp.kind == MlpSpec::NONE || dense_gemv_supported(pad_to(L.mlp.ff, 64)));
+        sc.attn = std::max(sc.attn, (size_t)rows * acols * eb);
+        const int fp = pad_to(L.mlp.ff, 64);
+        n.gemv = n.gemv && dense_gemv_supported(acols);
+        if (L.mlp.kind == MlpSpec::GATED_DENSE) {
+            sc.hmid = std::max(sc.hmid, (size_t)rows * fp * eb);
+            n.gemv = n.gemv && dense_gemv_supported(fp);
+        }
+        if (L.mlp.kind == MlpSpec::EXPERTS) {
+            scratch_experts(sc, L.mlp, c, ld);
+            n.gemv = n.gemv && expert_row_supported(ld, fp, L.mlp.top);
+        }
     }
     m.token_cap = c.max_seq + 8;
     ArenaPlan plan;
     const size_t o_xa = plan.take((size_t)rows * ld * 4), o_xb = plan.take((size_t)rows * ld * 4);
     const size_t o_x0 = plan.take(s.loop.times ? (size_t)rows * ld * 4 : 0);
-    const size_t o_act = plan.take((size_t)rows * ld * (s.loop.times ? 2 : 1) * eb), o_proj = plan.take(rows * n_in * eb);
-    const size_t o_attn = plan.take(rows * acols * eb), o_y = plan.take((size_t)rows * ld * eb), o_h = plan.take(rows * fp * eb);
-    const size_t o_qa = plan.take(q_abs * eb), o_po = plan.take(part_o * 4), o_pm = plan.take(part_ml * 4);
+    const size_t o_act = plan.take((size_t)rows * ld * (s.loop.times ? 2 : 1) * eb), o_proj = plan.take(sc.proj);
+    const size_t o_attn = plan.take(sc.attn), o_y = plan.take((size_t)rows * ld * eb), o_h = plan.take(sc.hmid);
+    const size_t o_qa = plan.take(q_abs * eb), o_po = plan.take(sc.part_o), o_pm = plan.take(sc.part_ml);
     const size_t o_c = plan.take(c_rows * eb), o_r = plan.take(rot_rows * eb), o_kv = plan.take(kv * eb);
     const size_t o_l = plan.take((size_t)rows * s.vocab * 4), o_sc = plan.take(32 + (size_t)c.batch * 4);
     const size_t o_ids = plan.take((size_t)rows * 8), o_pos = plan.take((size_t)c.seq_q * 8), o_tok = plan.take((size_t)m.token_cap * 4);
+    const size_t o_q = plan.take(sc.q), o_low = plan.take(sc.low), o_gates = plan.take(sc.gates), o_o = plan.take(sc.o), o_qk = plan.take(sc.qk);
+    const size_t o_v = plan.take(sc.v), o_scal = plan.take(sc.scal), o_dec = plan.take(sc.dec), o_rt = plan.take(sc.router), o_score = plan.take(sc.score);
+    const size_t o_parts = plan.take(sc.parts), o_chosen = plan.take(sc.chosen), o_choice = plan.take(sc.choice), o_tg = plan.take(sc.tile_group);
+    const size_t o_slot = plan.take(sc.slot), o_hs = plan.take(sc.hsort);
     const size_t o_ls = plan.take(4), o_cand = plan.take(kGreedyCands * sizeof(GreedyCand));
     m.arena_bytes = plan.off;
     MYNN_HIP(hipMalloc((void **)&m.arena, m.arena_bytes));
@@ -236,6 +248,10 @@ int build_layered(Model &m, void **state) {
     n.act = m.arena + o_act; n.proj = m.arena + o_proj; n.attn = m.arena + o_attn; n.y = m.arena + o_y; n.hmid = m.arena + o_h;
     n.q_abs = m.arena + o_qa; n.part_o = (float *)(m.arena + o_po); n.part_ml = (float *)(m.arena + o_pm);
     n.c_rows = m.arena + o_c; n.rot_rows = m.arena + o_r; n.kv = m.arena + o_kv;
+    n.q = m.arena + o_q; n.low = m.arena + o_low; n.gates = (float *)(m.arena + o_gates); n.o = (float *)(m.arena + o_o); n.qk = (float *)(m.arena + o_qk);
+    n.v = (float *)(m.arena + o_v); n.scal = (float *)(m.arena + o_scal); n.dec = (float *)(m.arena + o_dec); n.router = (float *)(m.arena + o_rt);
+    n.score = (float *)(m.arena + o_score); n.parts = (float *)(m.arena + o_parts); n.chosen = (int32_t *)(m.arena + o_chosen);
+    n.choice = (int32_t *)(m.arena + o_choice); n.tile_group = (int32_t *)(m.arena + o_tg); n.slot = (int32_t *)(m.arena + o_slot); n.hsort = m.arena + o_hs;
     m.logits = m.arena + o_l;
     m.d_past = (int32_t *)(m.arena + o_sc); m.d_active = m.d_past + 1; m.d_step = m.d_past + 2; m.d_next = m.d_past + 8;
     m.d_ids = (int64_t *)(m.arena + o_ids); m.d_pos = (int64_t *)(m.arena + o_pos); m.d_tokens = (int32_t *)(m.arena + o_tok);
@@ -250,27 +266,6 @@ int build_layered(Model &m, void **state) {
 }
 
 // ---- one step -------------------------------------------------------------------------------------------------------------
-namespace {
-// The residual stream of the step in flight: the current rows, and the sublayer output that the next linear's prologue
-// still has to norm and add.
-struct Stream {
-    Model &m;
-    LayeredNet &n;
-    int rows;
-    bool one;  // one row: the prologue rides on the linear (dense_gemv), which writes the sum to the other buffer
-    float *x, *other;
-    const void *y = nullptr, *wb = nullptr;
-
-    ResidualNorm row(const void *wa) const {
-        return ResidualNorm{x, y, wb, y ? (one ? other : x) : nullptr, wa, n.x0, n.spec->eps, n.spec->width, n.ld};
-    }
-    void added() {
-        if (y && one) std::swap(x, other);
-        y = wb = nullptr;
-    }
-    double row_bytes(double eb) const { return n.ld * (4 + (y ? 4 + 2 * eb : 0)); }
-};
-
 int linear(Stream &s, void *out, const DenseW &w, int store, const char *name, const char *gemv_name, const void *act, const void *wa, int pro) {
     const int dt = s.m.cfg.dtype;
     const double eb = dtype_size(dt), ob = store == DENSE_F32 ? 4 : eb, n_out = store == DENSE_GEGLU ? w.N / 2 : w.N;
@@ -291,7 +286,8 @@ int linear(Stream &s, void *out, const DenseW &w, int store, const char *name, c
     return dense_gemm(out, act, w.w, s.rows, w.N, w.K, store, nullptr, dt, s.m.stream);
 }
 
-// ---- mixers: act on n.proj / n.attn, leave the sublayer output in n.y
+namespace {
+// ---- latent attention: acts on n.proj / n.attn, leaves the sublayer output in n.y
 int latent_attention(Stream &st, int run, const LayerWeights &w, const MixerSpec &mix) {
     Model &m = st.m;
     LayeredNet &n = st.n;
@@ -371,10 +367,18 @@ int enqueue_layered(Model &m) {
             std::swap(st.x, st.other);
             st.y = st.wb = nullptr;
         }
-        TRY(latent_attention(st, (int)r, w, L.mixer));
+        if (L.mixer.kind == MixerSpec::PARALLEL) TRY(run_parallel(st, (int)r, w, L.mixer));
+        else if (L.mixer.kind == MixerSpec::CHANNEL_DELTA) TRY(run_channel_delta(st, (int)r, w, L.mixer));
+        else TRY(latent_attention(st, (int)r, w, L.mixer));
         st.y = n.y;
         st.wb = w.norm1b;
         if (L.mlp.kind == MlpSpec::NONE) continue;
+        if (L.mlp.kind == MlpSpec::EXPERTS) {
+            TRY(run_experts(st, w, L.mlp));
+            st.y = n.y;
+            st.wb = w.norm2b;
+            continue;
+        }
         TRY(linear(st, n.hmid, w.gu, DENSE_GEGLU, "linear_gateup_geglu", "gemv_norm_gateup_geglu", nullptr, w.norm2, PRO_RESIDUAL_NORM));
         TRY(linear(st, n.y, w.down, DENSE_T, "linear_down", "gemv_down", n.hmid, nullptr, PRO_ROWS));
         st.y = n.y;
@@ -418,5 +422,28 @@ int enqueue_layered(Model &m) {
     m.launches = (int)m.record.size();
     return 0;
 }
+
+// ---- a copy of the sequence states: what a run of the device loop computed past an end-of-sequence id is undone with it
+bool model_has_sequence_state(const void *state) {
+    const Model *m = (const Model *)state;
+    return m && m->net && m->net->spec->sequence_state();
+}
+static int copy_state(Model &m, bool save) {
+    LayeredNet &n = *m.net;
+    size_t off = 0, total = 0;
+    for (const StateSpec &st : n.spec->states) total += st.seq_floats * sizeof(float) * m.cfg.batch;
+    if (save && !n.saved) MYNN_HIP(hipMalloc((void **)&n.saved, total));
+    MYNN_REQUIRE(n.saved, MYNN_ERR_STATE, "sequence state: nothing saved");
+    for (size_t r = 0; r < n.spec->runs.size(); r++) {
+        if (!n.memory[r]) continue;
+        const size_t bytes = n.spec->states[n.spec->runs[r].memory].seq_floats * sizeof(float) * m.cfg.batch;
+        if (save) MYNN_HIP(hipMemcpyAsync(n.saved + off, n.memory[r], bytes, hipMemcpyDeviceToDevice, m.stream));
+        else MYNN_HIP(hipMemcpyAsync(n.memory[r], n.saved + off, bytes, hipMemcpyDeviceToDevice, m.stream));
+        off += bytes;
+    }
+    return 0;
+}
+int executor_save_state(void *state) { return copy_state(*(Model *)state, true); }
+int executor_restore_state(void *state) { return copy_state(*(Model *)state, false); }
 
 }  // namespace mynn

@@ -106,6 +106,7 @@ extern "C" mynn_llm *mynn_llm_create(void *decode_state, void *prefill_state, in
     l->prefill_len = prefill_state ? prefill_len : 0;
     l->max_seq = max_seq;
     l->eos = eos_token_id;
+    l->seq_state = model_has_sequence_state(decode_state);
     return l;
 }
 extern "C" mynn_llm *mynn_llm_create_with_step(mynn_step_fn step, void *user, int max_seq, int64_t eos_token_id) {
@@ -136,6 +137,13 @@ extern "C" void mynn_llm_reset(mynn_llm *l) {
 extern "C" int64_t mynn_llm_past_len(const mynn_llm *l) { return l ? l->past_len : -1; }
 extern "C" void mynn_llm_set_past_len(mynn_llm *l, int64_t p) { if (l) l->past_len = p < 0 ? 0 : p; }
 
+// A sequence state cannot be taken back to an earlier token: a call continues it where it is, or starts from position 0.
+static int check_state(const mynn_llm *l) {
+    MYNN_REQUIRE(!l->seq_state || l->past_len == 0 || l->past_len == l->state_len, MYNN_ERR_STATE,
+                 "the model's sequence state is behind %lld tokens and cannot continue from past_len %lld", (long long)l->state_len, (long long)l->past_len);
+    return 0;
+}
+
 // decode_step (session.rs:508-537): inputs [token, position = past_len, past_len, active = past_len + 1]
 static int decode_step(mynn_llm *l, int64_t token, int64_t *next) {
     if (l->step) {
@@ -160,6 +168,7 @@ static int decode_step(mynn_llm *l, int64_t token, int64_t *next) {
         *next = t;
     }
     l->past_len += 1;
+    l->state_len = l->past_len;
     return 0;
 }
 
@@ -180,6 +189,7 @@ static int run_prefill(mynn_llm *l, const int64_t *ids, size_t n, int64_t *next)
             int rc = mynn_model_step_rows(l->prefill, ids, (int)chunk, l->past_len, (int)chunk - 1, end ? 1 : 0, end ? &t : nullptr, nullptr);
             if (rc) return rc;
             l->past_len += (int64_t)chunk;
+            l->state_len = l->past_len;
             if (end) *next = t;
             ids += chunk;
             n -= chunk;
@@ -225,6 +235,8 @@ extern "C" int mynn_llm_feed(mynn_llm *l, const int64_t *ids, size_t n, const in
                      (long long)want[i], n);
     MYNN_REQUIRE(l->past_len + (int64_t)n <= l->max_seq, MYNN_ERR_TOO_LONG, "llm_feed: %lld + %zu tokens exceed max_seq %d", (long long)l->past_len, n,
                  l->max_seq);
+    int ok = check_state(l);
+    if (ok) return ok;
     const int V = mynn_model_vocab(l->decode);
     std::vector<float> span;
     size_t w = 0;
@@ -247,6 +259,7 @@ extern "C" int mynn_llm_feed(mynn_llm *l, const int64_t *ids, size_t n, const in
         w = w1;
         at += chunk;
         l->past_len += (int64_t)chunk;
+        l->state_len = l->past_len;
     }
     return 0;
 }
@@ -256,6 +269,8 @@ extern "C" int mynn_llm_generate_ids(mynn_llm *l, const int64_t *prompt_ids, siz
     MYNN_REQUIRE(l && (prompt_ids || n_prompt == 0) && (out || max_new_tokens == 0), MYNN_ERR_INVALID,
                  "llm_generate_ids: null argument");
     if (n_prompt == 0) return 0;
+    int ok = check_state(l);
+    if (ok) return ok;
     const bool prefill_runs = l->prefill != nullptr;
     const int64_t needed = prefill_runs && !model_takes_any_rows(l->prefill)
         ? l->past_len + (int64_t)((n_prompt + l->prefill_len - 1) / l->prefill_len * l->prefill_len)
@@ -265,7 +280,8 @@ extern "C" int mynn_llm_generate_ids(mynn_llm *l, const int64_t *prompt_ids, siz
     int n_new = 0;
     // the executor's device-resident loop (mynn_model_decode_loop) serves runs of decode steps without a host round
     // trip per token; with an end-of-sequence id the runs are short, and what a run computed past that id is dropped
-    // (its cache rows lie beyond past_len, where the next turn overwrites them)
+    // (its cache rows lie beyond past_len, where the next turn overwrites them; a sequence state is saved before a run that
+    // may have to be cut, and then taken through the tokens that count)
     bool loop_ok = !l->step && !l->streaming && l->decode != nullptr;
     std::vector<int32_t> run;
     for (size_t i = 0; i < max_new_tokens;) {
@@ -283,13 +299,22 @@ extern "C" int mynn_llm_generate_ids(mynn_llm *l, const int64_t *prompt_ids, siz
             const size_t want = std::min<size_t>(std::min<size_t>(max_new_tokens - i, l->eos >= 0 ? 32 : 256), (size_t)room);
             if (loop_ok && want >= 4) {
                 run.resize(want);
-                if (mynn_model_decode_loop(l->decode, out[n_new - 1], l->past_len, (int)want, run.data()) == 0) {
+                const int32_t first = (int32_t)out[n_new - 1];
+                const bool cut = l->seq_state && l->eos >= 0;
+                if (cut && (rc = executor_save_state(l->decode))) return rc;
+                if (mynn_model_decode_loop(l->decode, first, l->past_len, (int)want, run.data()) == 0) {
                     size_t used = 0;
                     while (used < want) {
                         out[n_new++] = run[used++];
                         if (out[n_new - 1] == l->eos) break;
                     }
+                    if (cut && used < want) {
+                        rc = executor_restore_state(l->decode);
+                        if (!rc) rc = mynn_model_decode_loop(l->decode, first, l->past_len, (int)used, run.data());
+                        if (rc) return rc;
+                    }
                     l->past_len += (int64_t)used;
+                    l->state_len = l->past_len;
                     i += used;
                     if (out[n_new - 1] == l->eos) break;
                     continue;

@@ -11,6 +11,9 @@ struct mynn_llm {
     int last_error = 0;
     void (*release)(mynn_llm *) = nullptr;  // an engine's session: gives its executors and cache back
     void *owner = nullptr;
+    // models with a sequence state (recurrences): it stands for the first state_len tokens, and only they can be continued
+    bool seq_state = false;
+    int64_t state_len = 0;
     bool streaming = false;  // DecodeKind::LlamaStreaming { sink, window }
     int sink = 0, window = 0;
 };
