@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Headline benchmark: batch-1 greedy decode of a TinyLlama-1.1B-shape int8 model on one MI355X.
 
-  python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload decode|prefill|attention|decode_batch|gemv|latent]
+  python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload decode|prefill|attention|decode_batch|gemv|latent|recurrent]
 
 `--workload prefill` times the matrix-core side of the same path instead: one step = one prefill
 pass of 8 prompts x 1024 tokens through the decoder executor (roofline bound: MFMA).
@@ -827,6 +827,42 @@ LATENT_PAIRS = {
 }
 
 
+def per_kernel(profile, reps, kv_bytes, block_names=()):
+    """launch name -> time, bound and fraction of the roofline; block_names: launches summed up as attention_block"""
+    agg = {}
+    for _ in range(reps):
+        for name, ms, nbytes, flops in profile():
+            a = agg.setdefault(name, [0, 0.0, 0.0, 0.0])
+            a[0] += 1
+            a[1] += ms
+            a[2] += nbytes + kv_bytes.get(name, 0.0)
+            a[3] += flops
+    out = {}
+    block = [v for k, v in agg.items() if k in block_names]
+    if kv_bytes and block:
+        agg["attention_block"] = [max(v[0] for v in block)] + [sum(v[i] for v in block) for i in (1, 2, 3)]
+    for name, (n, ms, nb, fl) in agg.items():
+        t = ms * 1e-3
+        if t <= 0:
+            continue
+        hbm, mfma = nb / t / 1e9 / HBM_PEAK_GBS, fl / t / 1e12 / MFMA_PEAK_TFLOPS
+        out[name] = {"us": round(t / n * 1e6, 2), "per_step": n // reps, "bound": "hbm" if hbm >= mfma else "mfma", "frac": round(max(hbm, mfma), 4)}
+    return out
+
+
+def rate(fn, n, warm):
+    import torch
+
+    for _ in range(warm):
+        fn()
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(n):
+        fn()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / n
+
+
 def latent_config(size):
     H = size["heads"]
     mix = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
@@ -851,37 +887,6 @@ def latent_main(args, mynn):
     gen.manual_seed(args.seed)
     rng = np.random.default_rng(args.seed)
 
-    def per_kernel(profile, reps, kv_bytes):
-        agg = {}
-        for _ in range(reps):
-            for name, ms, nbytes, flops in profile():
-                a = agg.setdefault(name, [0, 0.0, 0.0, 0.0])
-                a[0] += 1
-                a[1] += ms
-                a[2] += nbytes + kv_bytes.get(name, 0.0)
-                a[3] += flops
-        out = {}
-        block = [v for k, v in agg.items() if k in LATENT_ATTENTION_BLOCK]
-        if kv_bytes:
-            agg["attention_block"] = [max(v[0] for v in block)] + [sum(v[i] for v in block) for i in (1, 2, 3)]
-        for name, (n, ms, nb, fl) in agg.items():
-            t = ms * 1e-3
-            if t <= 0:
-                continue
-            hbm, mfma = nb / t / 1e9 / HBM_PEAK_GBS, fl / t / 1e12 / MFMA_PEAK_TFLOPS
-            out[name] = {"us": round(t / n * 1e6, 2), "per_step": n // reps, "bound": "hbm" if hbm >= mfma else "mfma", "frac": round(max(hbm, mfma), 4)}
-        return out
-
-    def rate(fn, n, warm):
-        for _ in range(warm):
-            fn()
-        torch.cuda.synchronize()
-        t0 = time.perf_counter()
-        for _ in range(n):
-            fn()
-        torch.cuda.synchronize()
-        return (time.perf_counter() - t0) / n
-
     sizes = {}
     for label, size in LATENT_SIZES.items():
         ids = rng.integers(0, size["vocab"], ctx)
@@ -905,8 +910,8 @@ def latent_main(args, mynn):
         row = (512 + 64) * 2.0  # cached bytes of a token and layer run
         res["latent"] = {"prefill_tok_s": round(ctx / t_pre), "decode_tok_s": round(1 / t_dec, 1), "launches_per_step": dec.stats()["launches_per_step"],
                          "prefill": per_kernel(lambda: pre.profile(ids, pos, 0, ctx), 3, {}),
-                         "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, {"latent_attention": (ctx + 33) * row}),
-                         "decode_far": per_kernel(lambda: dec.profile_step(1, far + 32), 8, {"latent_attention": (far + 33) * row})}
+                         "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, {"latent_attention": (ctx + 33) * row}, LATENT_ATTENTION_BLOCK),
+                         "decode_far": per_kernel(lambda: dec.profile_step(1, far + 32), 8, {"latent_attention": (far + 33) * row}, LATENT_ATTENTION_BLOCK)}
         dec.decode_loop(1, far, W)
         res["latent"]["decode_far_tok_s"] = round(K / rate(lambda: dec.decode_loop(1, far, K), 3, 1), 1)
         pre.close(), dec.close()
@@ -924,8 +929,8 @@ def latent_main(args, mynn):
         kv = lambda n: {k: (n + 33) * 2.0 * cfg["n_kv_heads"] * 128 * 2 for k in ("attention_rope_append", "attention")}
         res["llama"] = {"prefill_tok_s": round(ctx / t_pre), "decode_tok_s": round(1 / t_dec, 1), "launches_per_step": dec.stats()["launches_per_step"],
                         "prefill": per_kernel(lambda: pre.profile(ids, pos, 0, ctx), 3, {}),
-                        "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, kv(ctx)),
-                        "decode_far": per_kernel(lambda: dec.profile_step(1, far + 32), 8, kv(far))}
+                        "decode": per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, kv(ctx), LATENT_ATTENTION_BLOCK),
+                        "decode_far": per_kernel(lambda: dec.profile_step(1, far + 32), 8, kv(far), LATENT_ATTENTION_BLOCK)}
         dec.decode_loop(1, far, W)
         res["llama"]["decode_far_tok_s"] = round(K / rate(lambda: dec.decode_loop(1, far, K), 3, 1), 1)
         pre.close(), dec.close()
@@ -953,10 +958,147 @@ def latent_main(args, mynn):
                      "achieved": round(last["decode"][dom]["frac"] * HBM_PEAK_GBS, 1), "avg_launch_us": last["decode"][dom]["us"]}}))
 
 
+# --workload recurrent: layers of the sizes real models have, the recurrent design (delta rule and parallel mixers in turn, 6
+# layers, two of eight experts per token) beside the latent-attention design (6 layers, one dense feed-forward of the two
+# experts' size) at equal width, heads and vocabulary; bf16 weights on both sides
+RECURRENT_SIZES = {
+    "2048": dict(width=2048, heads=16, ff=2816, vocab=32000),
+    "3072": dict(width=3072, heads=24, ff=4096, vocab=64000),
+    "4096": dict(width=4096, heads=32, ff=7168, vocab=128256),
+}
+RECURRENT_WINDOW, RECURRENT_KEEP, RECURRENT_RANK = 2048, 4, 128
+# launch of the design -> the like launch of the latent-attention design.  A recurrence reads and writes its state where an
+# attention reads its cache: its decode launch is set beside the whole attention block.
+RECURRENT_BLOCK = ("attention_prepare_memory_step", "window_attention", "window_merge")
+RECURRENT_PAIRS = {
+    "decode": {"gemv_delta_in": "gemv_norm_latent_in", "gemv_parallel_in": "gemv_norm_latent_in", "gemv_o": "gemv_o",
+               "gemv_experts_gateup": "gemv_norm_gateup_geglu", "gemv_experts_down": "gemv_down", "window_attention": "latent_attention",
+               "attention_block": "attention_block", "delta_step": "attention_block", "gemv_norm_head": "gemv_norm_head"},
+    "prefill": {"linear_delta_in": "linear_latent_in", "linear_parallel_in": "linear_latent_in", "linear_o": "linear_o",
+                "linear_experts_gateup": "linear_gateup_geglu", "linear_experts_down": "linear_down", "window_attention": "latent_attention",
+                "residual_norm": "residual_norm", "attention_prepare": "latent_rotate_append", "delta_prepare": "latent_rotate_append",
+                "head_norm_gate": "residual_norm", "linear_delta_low": "linear_latent_kv"},
+}
+
+
+def recurrent_config(size):
+    H = size["heads"]
+    moe = {"kind": "moe", "expert": {"ff": size["ff"]}, "router": {"experts": 8, "top": 2}}
+    delta = {"type": "channel_delta", "mlp": moe, "mixer": {"heads": H, "kv_heads": H // 2, "dim": 128, "vdim": 128, "conv": 4}}
+    rot = {"base": 500000.0, "dims": 128, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}
+    left = {"heads": H, "kv_heads": H // 4, "dim": 128, "vdim": 128, "conv": 4, "scale": 128 ** -0.5, "rot": rot,
+            "mask": {"size": RECURRENT_WINDOW, "keep_first": RECURRENT_KEEP}}
+    par = {"type": "parallel", "mlp": moe, "mixer": {"left": left, "right": {"heads": H // 2, "dim": 128, "vdim": 128, "gate_cap": 15.0},
+                                                     "left_scale": 0.7, "right_scale": 0.9}}
+    return {"architecture": "Kulanex", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-5}, "residual_mult": 0.3,
+            "layers": [delta, par] * 3}
+
+
+def recurrent_arch(mynn, size):
+    """the design's config, with a checkpoint that holds the tensors whose rows the config leaves open"""
+    import struct
+    import tempfile
+
+    with tempfile.TemporaryDirectory() as d:
+        with open(os.path.join(d, "config.json"), "w") as f:
+            json.dump(recurrent_config(size), f)
+        n = RECURRENT_RANK * size["width"] * 2
+        names = ["l%d.mix.%s" % (i, t) for i in (0, 2, 4) for t in ("a1", "g1")]
+        head = json.dumps({t: {"dtype": "BF16", "shape": [RECURRENT_RANK, size["width"]], "data_offsets": [i * n, (i + 1) * n]} for i, t in enumerate(names)}).encode()
+        with open(os.path.join(d, "model.safetensors"), "wb") as f:
+            f.write(struct.pack("<Q", len(head)) + head + bytes(n * len(names)))
+        return mynn.Arch(d)
+
+
+def layered_weights(arch, gen):
+    import torch
+
+    out = {}
+    for name, sh in arch.tensors():
+        last = name.split(".")[-1]
+        if len(sh) == 1:
+            fill = {"A_log": -2.0, "dt_bias": -2.0, "norm1": 0.0, "norm2": 0.0}.get(last, 4.0 if name.endswith("f.b") else 0.0 if name.endswith("i.b") else 1.0)
+            out[name] = torch.full(sh, fill, dtype=torch.bfloat16, device="cuda")
+        else:
+            out[name] = (torch.randn(sh, generator=gen, device="cuda") * (1.0 if name in ("embed", "bigram") else sh[1] ** -0.5)).to(torch.bfloat16)
+    return out
+
+
+def recurrent_main(args, mynn):
+    """Prefill of one prompt and batch-1 decode behind it, bf16, random weights: tokens/s of both designs and, per launch, the
+    distance from the roofline beside the like launch of the latent-attention design."""
+    import tempfile
+
+    import numpy as np
+    import torch
+
+    ctx, K, W = 2048, args.steps or 64, args.warmup or 16
+    far = 16384
+    max_seq = far + 256
+    gen = torch.Generator(device="cuda")
+    gen.manual_seed(args.seed)
+    rng = np.random.default_rng(args.seed)
+    labels = [args.size] if args.size else list(RECURRENT_SIZES)
+    sizes = {}
+    for label in labels:
+        size = RECURRENT_SIZES[label]
+        ids = rng.integers(0, size["vocab"], ctx)
+        pos = np.arange(ctx)
+        res = {}
+        sees = lambda n: min(n, RECURRENT_WINDOW + RECURRENT_KEEP)
+        row = 2.0 * (size["heads"] // 4) * 128 * 2
+        designs = {"recurrent": (lambda: recurrent_arch(mynn, size), lambda n: {"window_attention": sees(n + 33) * row}, RECURRENT_BLOCK),
+                   "latent": (None, lambda n: {"latent_attention": (n + 33) * (512 + 64) * 2.0}, LATENT_ATTENTION_BLOCK)}
+        for name, (make, kv, block) in designs.items():
+            if make:
+                arch = make()
+            else:
+                cfg = latent_config(dict(size, ff=2 * size["ff"]))
+                with tempfile.TemporaryDirectory() as d:
+                    with open(os.path.join(d, "config.json"), "w") as f:
+                        json.dump(cfg, f)
+                    arch = mynn.Arch(d)
+            w = layered_weights(arch, gen)
+            state = mynn.layered_state(arch, mynn.BF16, max_seq)
+            pre = mynn.LayeredDecoder(arch, w, mynn.BF16, max_seq, seq_q=ctx, state=state)
+            dec = mynn.LayeredDecoder(arch, w, mynn.BF16, max_seq, state=state)
+            r = {"prefill_tok_s": round(ctx / rate(lambda: pre.step_rows(ids, ctx, 0), 5, 2))}
+            dec.decode_loop(1, ctx, W)
+            r["decode_tok_s"] = round(K / rate(lambda: dec.decode_loop(1, ctx, K), 3, 1), 1)
+            r["launches_per_step"] = dec.stats()["launches_per_step"]
+            r["prefill"] = per_kernel(lambda: pre.profile(ids, pos, 0, ctx), 3, {})
+            r["decode"] = per_kernel(lambda: dec.profile_step(1, ctx + 32), 8, kv(ctx), block)
+            r["decode_far"] = per_kernel(lambda: dec.profile_step(1, far + 32), 8, kv(far), block)
+            dec.decode_loop(1, far, W)
+            r["decode_far_tok_s"] = round(K / rate(lambda: dec.decode_loop(1, far, K), 3, 1), 1)
+            res[name] = r
+            pre.close(), dec.close()
+            del w, state
+            torch.cuda.empty_cache()
+        # distance from the roofline relative to the like launch's: 1 / frac against 1 / frac
+        for phase, pairs in list(RECURRENT_PAIRS.items()) + [("decode_far", RECURRENT_PAIRS["decode"])]:
+            res["times_farther_" + phase] = {mine: [like, round(res["latent"][phase][like]["frac"] / max(res["recurrent"][phase][mine]["frac"], 1e-6), 2)]
+                                             for mine, like in pairs.items() if mine in res["recurrent"][phase] and like in res["latent"][phase]}
+        sizes[label] = res
+        print("bench.py: recurrent %s done" % label, file=sys.stderr, flush=True)
+    last = sizes[labels[-1]]["recurrent"]
+    dom = max(last["decode"], key=lambda k: last["decode"][k]["us"] * last["decode"][k]["per_step"])
+    print(json.dumps({
+        "metric": "decode tok/s behind %d tokens, recurrent design, width %s, 6 layers" % (ctx, labels[-1]), "value": last["decode_tok_s"], "unit": "tok/s",
+        "n_gpus": 1, "steps": K, "warmup": W, "ms_per_step": round(1e3 / last["decode_tok_s"], 4), "higher_is_better": True, "scaling": "weak",
+        "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "delta rule (dim 128) and window attention (%d + %d kept) beside a matrix memory (dim 128) in turn, 2 of 8 experts, beside the "
+                               "latent-attention design at equal sizes; prompt of %d tokens, then decode" % (RECURRENT_WINDOW, RECURRENT_KEEP, ctx),
+                   "seed": args.seed, "sizes": sizes},
+        "roofline": {"bound": last["decode"][dom]["bound"], "kernel": dom, "frac": last["decode"][dom]["frac"], "peak": HBM_PEAK_GBS, "unit": "GB/s",
+                     "achieved": round(last["decode"][dom]["frac"] * HBM_PEAK_GBS, 1), "avg_launch_us": last["decode"][dom]["us"]}}))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
-    ap.add_argument("--workload", choices=["decode", "prefill", "attention", "decode_batch", "gemv", "latent"], default="decode")
+    ap.add_argument("--workload", choices=["decode", "prefill", "attention", "decode_batch", "gemv", "latent", "recurrent"], default="decode")
+    ap.add_argument("--size", choices=list(RECURRENT_SIZES), default=None, help="recurrent: this width only")
     ap.add_argument("--steps", type=int, default=None, help="default 256 (decode) / 5 (prefill)")
     ap.add_argument("--warmup", type=int, default=None, help="default 16 (decode) / 2 (prefill)")
     ap.add_argument("--dtype", choices=["f16", "bf16"], default="f16")
@@ -1022,6 +1164,8 @@ def main():
         return gemv_main(args, mynn)
     if args.workload == "latent":
         return latent_main(args, mynn)
+    if args.workload == "recurrent":
+        return recurrent_main(args, mynn)
     K = 256 if args.steps is None else args.steps
     W = 16 if args.warmup is None else args.warmup
     # the cache of configs[2] holds 128 + 256 rows; longer runs get a longer cache (whole 128-row pages, up to the 2048 rows

@@ -53,7 +53,7 @@ struct LayeredNet {
     bool gemv = false;            // every linear fits the one-row kernel
     // recurrent mixers and window attention
     void *q = nullptr, *low = nullptr;
-    float *gates = nullptr, *o = nullptr, *qk = nullptr, *v = nullptr, *scal = nullptr, *dec = nullptr;
+    float *gates = nullptr, *o = nullptr, *qk = nullptr, *v = nullptr, *beta = nullptr, *dec = nullptr, *blocks = nullptr;
     // experts
     float *router = nullptr, *score = nullptr, *parts = nullptr;
     int32_t *chosen = nullptr, *choice = nullptr, *tile_group = nullptr, *slot = nullptr;
@@ -91,7 +91,7 @@ int pack_experts(WeightPacker &pk, LayerWeights &o, const MlpSpec &mlp, const st
 // bytes of the buffers the mixers need, the most of any layer
 struct MixerScratch {
     size_t proj = 0, attn = 0, part_o = 0, part_ml = 0;
-    size_t q = 0, low = 0, gates = 0, o = 0, qk = 0, v = 0, scal = 0, dec = 0;
+    size_t q = 0, low = 0, gates = 0, o = 0, qk = 0, v = 0, beta = 0, dec = 0, blocks = 0;
     size_t hmid = 0, router = 0, score = 0, parts = 0, chosen = 0, choice = 0, tile_group = 0, slot = 0, hsort = 0;
 };
 void scratch_recurrent(MixerScratch &x, const MixerSpec &mix, const mynn_model_config &c);

@@ -237,7 +237,7 @@ int build_layered(Model &m, void **state) {
     const size_t o_l = plan.take((size_t)rows * s.vocab * 4), o_sc = plan.take(32 + (size_t)c.batch * 4);
     const size_t o_ids = plan.take((size_t)rows * 8), o_pos = plan.take((size_t)c.seq_q * 8), o_tok = plan.take((size_t)m.token_cap * 4);
     const size_t o_q = plan.take(sc.q), o_low = plan.take(sc.low), o_gates = plan.take(sc.gates), o_o = plan.take(sc.o), o_qk = plan.take(sc.qk);
-    const size_t o_v = plan.take(sc.v), o_scal = plan.take(sc.scal), o_dec = plan.take(sc.dec), o_rt = plan.take(sc.router), o_score = plan.take(sc.score);
+    const size_t o_v = plan.take(sc.v), o_beta = plan.take(sc.beta), o_bl = plan.take(sc.blocks), o_dec = plan.take(sc.dec), o_rt = plan.take(sc.router), o_score = plan.take(sc.score);
     const size_t o_parts = plan.take(sc.parts), o_chosen = plan.take(sc.chosen), o_choice = plan.take(sc.choice), o_tg = plan.take(sc.tile_group);
     const size_t o_slot = plan.take(sc.slot), o_hs = plan.take(sc.hsort);
     const size_t o_ls = plan.take(4), o_cand = plan.take(kGreedyCands * sizeof(GreedyCand));
@@ -249,7 +249,7 @@ int build_layered(Model &m, void **state) {
     n.q_abs = m.arena + o_qa; n.part_o = (float *)(m.arena + o_po); n.part_ml = (float *)(m.arena + o_pm);
     n.c_rows = m.arena + o_c; n.rot_rows = m.arena + o_r; n.kv = m.arena + o_kv;
     n.q = m.arena + o_q; n.low = m.arena + o_low; n.gates = (float *)(m.arena + o_gates); n.o = (float *)(m.arena + o_o); n.qk = (float *)(m.arena + o_qk);
-    n.v = (float *)(m.arena + o_v); n.scal = (float *)(m.arena + o_scal); n.dec = (float *)(m.arena + o_dec); n.router = (float *)(m.arena + o_rt);
+    n.v = (float *)(m.arena + o_v); n.beta = (float *)(m.arena + o_beta); n.blocks = (float *)(m.arena + o_bl); n.dec = (float *)(m.arena + o_dec); n.router = (float *)(m.arena + o_rt);
     n.score = (float *)(m.arena + o_score); n.parts = (float *)(m.arena + o_parts); n.chosen = (int32_t *)(m.arena + o_chosen);
     n.choice = (int32_t *)(m.arena + o_choice); n.tile_group = (int32_t *)(m.arena + o_tg); n.slot = (int32_t *)(m.arena + o_slot); n.hsort = m.arena + o_hs;
     m.logits = m.arena + o_l;

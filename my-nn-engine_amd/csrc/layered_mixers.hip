@@ -109,6 +109,7 @@ void scratch_recurrent(MixerScratch &x, const MixerSpec &mix, const mynn_model_c
         if (many) {
             grow(x.gates, rows * d.R * 16);
             grow(x.o, rows * d.R * pad_to(d.rv + 1, 4) * 4);
+            grow(x.blocks, recurrent_block_floats(c.batch, c.seq_q, d.R, d.rdp, false) * 4);
         }
     } else if (mix.kind == MixerSpec::CHANNEL_DELTA) {
         const DeltaDims d = delta_dims(mix.delta);
@@ -116,7 +117,8 @@ void scratch_recurrent(MixerScratch &x, const MixerSpec &mix, const mynn_model_c
         if (!many) return;
         grow(x.qk, rows * 2 * d.G * d.dp * 4);
         grow(x.v, rows * d.H * d.vp * 4);
-        grow(x.scal, rows * (d.H + d.G) * 4);
+        grow(x.beta, rows * d.H * 4);
+        grow(x.blocks, recurrent_block_floats(c.batch, c.seq_q, d.H, d.dp, true) * 4);
         grow(x.low, rows * d.low() * eb);
         grow(x.dec, rows * d.n_low() * 4);
         grow(x.o, rows * d.H * d.vp * 4);
@@ -154,7 +156,7 @@ int run_parallel(Stream &st, int run, const LayerWeights &w, const MixerSpec &mi
     MemoryParams r{};
     r.d = d; r.cap = mix.memory.gate_cap; r.out_scale = mix.right_scale; r.eps = n.spec->eps; r.q_scale = 1.0f / sqrtf((float)d.rd);
     r.proj = (const float *)n.proj; r.i_bias = w.i_bias; r.f_bias = w.f_bias; r.norm = w.head_norm; r.state = n.memory[run]; r.state_stride = d.state();
-    r.d_past = m.d_past; r.B = B; r.S = S; r.out = n.attn; r.gates = n.gates; r.o = n.o;
+    r.d_past = m.d_past; r.B = B; r.S = S; r.out = n.attn; r.gates = n.gates; r.o = n.o; r.blocks = n.blocks;
     const double prep = rows * (d.conv() * 4.0 + (d.qcols() + d.row()) * eb), mem = 2.0 * B * d.st_max() * 4.0, memio = rows * d.R * (2.0 * d.rdp + d.rvp) * 4;
     note(m, S == 1 ? "attention_prepare_memory_step" : "attention_prepare", S == 1 ? prep + mem + memio + rows * d.R * d.rvp * (4 + eb) : prep + rows * d.R * 24.0);
     TRY(parallel_prepare(a, r, c.dtype, m.stream));
@@ -175,7 +177,10 @@ int run_parallel(Stream &st, int run, const LayerWeights &w, const MixerSpec &mi
         }
     }
     if (S > 1) {
-        note(m, "memory_recurrence", memio + mem + rows * d.R * (d.rv + 1) * 4.0, 6.0 * rows * d.R * d.rd * (d.rv + 1));
+        const double ops = recurrent_block_floats(B, S, d.R, d.rdp, false) * 4.0;
+        note(m, "memory_blocks", rows * d.R * 2.0 * d.rdp * 4 + ops);
+        TRY(memory_blocks(r, m.stream));
+        note(m, "memory_recurrence", ops + mem + rows * d.R * (d.rvp + d.rv + 1.0) * 4, 4.0 * rows * d.R * (d.rd + 8) * (d.rv + 1));
         TRY(memory_recurrence(r, m.stream));
         note(m, "head_norm_gate", rows * d.R * d.rvp * (8.0 + eb));
         TRY(memory_out(a, r, c.dtype, m.stream));
@@ -194,7 +199,7 @@ int run_channel_delta(Stream &st, int run, const LayerWeights &w, const MixerSpe
     DeltaParams p{};
     p.d = d; p.eps = n.spec->eps; p.proj = (const float *)n.proj; p.conv_w = w.taps; p.low_w = w.low.w; p.a_log = w.a_log; p.dt_bias = w.dt_bias;
     p.norm = w.head_norm; p.state = n.memory[run]; p.state_stride = d.state(); p.d_past = m.d_past; p.B = B; p.S = S; p.out = n.attn;
-    p.qk = n.qk; p.v = n.v; p.scal = n.scal; p.low = n.low; p.dec = n.dec; p.o = n.o;
+    p.qk = n.qk; p.v = n.v; p.beta = n.beta; p.blocks = n.blocks; p.low = n.low; p.dec = n.dec; p.o = n.o;
     const double state = 2.0 * B * d.H * d.v * d.dp * 4.0;
     if (S == 1) {
         note(m, "delta_step", state + (double)w.low.N * w.low.K * eb / 2 + rows * (d.n_in() * 4.0 + d.acols() * eb + 2.0 * d.taps * d.conv() * 4));
@@ -204,9 +209,10 @@ int run_channel_delta(Stream &st, int run, const LayerWeights &w, const MixerSpe
         TRY(delta_prepare(p, c.dtype, m.stream));
         note(m, "linear_delta_low", ((double)w.low.N * w.low.K + rows * w.low.K) * eb + rows * w.low.N * 4, 2.0 * rows * w.low.N * w.low.K);
         TRY(dense_gemm(n.dec, n.low, w.low.w, st.rows, w.low.N, w.low.K, DENSE_F32, nullptr, c.dtype, m.stream));
-        note(m, "delta_decays", rows * d.H * d.dp * 8.0);
-        TRY(delta_decays(p, c.dtype, m.stream));
-        note(m, "delta_recurrence", state + rows * (2.0 * d.G * d.dp + d.H * (d.dp + 2.0 * d.vp)) * 4, 9.0 * rows * d.H * d.d * d.v);
+        const double ops = recurrent_block_floats(B, S, d.H, d.dp, true) * 4.0;
+        note(m, "delta_blocks", rows * (2.0 * d.G * d.dp + d.H * d.dp) * 4 + ops);
+        TRY(delta_blocks(p, c.dtype, m.stream));
+        note(m, "delta_recurrence", state + ops + rows * d.H * 2.0 * d.vp * 4, 6.0 * rows * d.H * (d.d + 11) * d.v);
         TRY(delta_recurrence(p, m.stream));
         note(m, "head_norm_gate", rows * d.H * d.vp * (8.0 + eb));
         TRY(delta_out(p, c.dtype, m.stream));

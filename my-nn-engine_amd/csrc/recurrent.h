@@ -7,6 +7,10 @@ namespace mynn {
 
 // state rows [dp] of key channels, one per value column: a column is its own recurrence given the keys, queries and gates
 bool recurrent_dim_supported(int dp);
+// several tokens: blocks of kRecurrentBlock tokens, key channels padded to whole operand tiles; floats of a portion's operands
+constexpr int kRecurrentBlock = 16;
+__host__ __device__ inline int recurrent_keys(int dp) { return dp <= 64 ? 64 : dp <= 128 ? 128 : dp <= 256 ? 256 : 512; }
+size_t recurrent_block_floats(int B, int S, int H, int dp, bool delta);
 
 struct DeltaParams {
     DeltaDims d;
@@ -23,14 +27,15 @@ struct DeltaParams {
     // several tokens at a time: prepared operands of the recurrence
     float *qk;                // [B * S, 2 * G * dp] unit queries | keys
     float *v;                 // [B * S, H * vp]
-    float *scal;              // [B * S, H + G]: beta per head, then q . k per key head
+    float *beta;              // [B * S, H]
     void *low;                // T [B * S, low()]
-    float *dec;               // [B * S, n_low()]: decays | gates before their sigmoid
+    float *dec;               // [B * S, n_low()]: decays | gates, as the second map leaves them
+    float *blocks;            // recurrent_block_floats
     float *o;                 // [B * S, H * vp]
 };
 int delta_step(const DeltaParams &p, int dtype, hipStream_t s);      // one new token per sequence: all of the mixer between its projections
 int delta_prepare(const DeltaParams &p, int dtype, hipStream_t s);   // convolutions, unit norms, beta; low
-int delta_decays(const DeltaParams &p, int dtype, hipStream_t s);    // dec: the second map's output -> decays
+int delta_blocks(const DeltaParams &p, int dtype, hipStream_t s);    // decays; the operands of every block
 int delta_recurrence(const DeltaParams &p, hipStream_t s);
 int delta_out(const DeltaParams &p, int dtype, hipStream_t s);       // head norm and gate; the conv ring
 
@@ -44,12 +49,14 @@ struct MemoryParams {
     const int32_t *d_past;
     int B, S;
     void *out;                // T [B * S, acols()], heads behind the attention's
+    float *blocks;            // recurrent_block_floats
     float *gates;             // [B * S, R, 4]: what is kept, what is put in, exp(-maximum)
     float *o;                 // [B * S, R, pad4(rv + 1)]: unnormed read-out, then the normaliser's
 };
 // both mixers of a parallel layer: convolutions, norms, rotation and cache append of the attention; for one new token per
 // sequence the whole memory step, else the memory's gates
 int parallel_prepare(const WindowAttnParams &a, const MemoryParams &m, int dtype, hipStream_t s);
+int memory_blocks(const MemoryParams &p, hipStream_t s);
 int memory_recurrence(const MemoryParams &p, hipStream_t s);
 int memory_out(const WindowAttnParams &a, const MemoryParams &p, int dtype, hipStream_t s);  // head norm and gate; the attention's conv ring
 

@@ -3,9 +3,14 @@
 //
 // One new token: delta_step_kernel / the memory workgroups of parallel_prepare_kernel, one workgroup per head, do everything
 // between the two projections; the first state columns are requested before anything else.
-// Several tokens: the elementwise parts run over all rows at once, then recurrence_kernel walks the tokens.  A column's key
-// channels are spread over LC lanes, RP per lane, in registers; keys, queries and decays of a chunk of tokens come through
-// LDS, shared by the waves of a workgroup, with the next chunk in registers meanwhile.
+// Several tokens: the elementwise parts run over all rows at once, then the tokens go through the recurrence sixteen at a time.
+// With S the state in front of a block, G_j the product of its decays up to token j, and u_i what token i writes,
+//     u_j = beta_j (v_j - (G_j k_j) . S - sum_{i<j} A_ji u_i),  A_ji = k_j . (g_{i+1} .. g_j k_i)
+//     o_j = (G_j q_j) . S + sum_{i<=j} B_ji u_i,                B_ji = q_j . (g_{i+1} .. g_j k_i)
+//     S  <- G_16 S + sum_i (g_{i+1} .. g_16 k_i) u_i
+// (products of decays only, no quotients).  What does not depend on the values -- G k, G q, the keys carried to the block's
+// end, B and the inverse T of the triangular system -- is made for all blocks in parallel (delta_blocks_kernel,
+// memory_blocks_kernel, whose u_i is the value itself); recurrence_kernel then walks the blocks with f32 matrix-core products.
 #include <algorithm>
 #include <type_traits>
 
@@ -256,29 +261,29 @@ __device__ inline void memory_step(const MemoryParams &p, int head, int b, float
                                            sigmoidf(proj[d.mem_g() + head * d.rvp + c]) * p.out_scale : 0.f);
 }
 
-// Gates of all tokens of a portion, one wave per (sequence, head): input and forget gates one token per lane, the running
-// maximum token by token.
+// Gates of all tokens of a portion, one wave per (sequence, head).  The running maximum is a scan over maps
+// m -> max(f + m, i), 64 tokens at a time.  (A maximum that is off by a rounding scales state, normaliser and floor alike.)
 template <typename T> __device__ inline void memory_gate_scan(const MemoryParams &p, int head, int b) {
     const ParallelDims &d = p.d;
     const int lane = threadIdx.x & 63;
     float *mx = p.state + (size_t)b * p.state_stride + d.st_max() + head;
     float m = *p.d_past ? *mx : 0.f;
     for (int t0 = 0; t0 < p.S; t0 += 64) {
+        const int n = min(64, p.S - t0);
         const size_t row = (size_t)b * p.S + min(t0 + lane, p.S - 1);
         const MemoryGates gt = memory_gates<T>(p, p.proj + row * d.n_in(), head);
-        float before = 0.f, after = 0.f;
-        const int n = min(64, p.S - t0);
-        for (int j = 0; j < n; j++) {
-            const float f = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, gt.forget), j));
-            const float i = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, gt.in), j));
-            const float mn = fmaxf(f + m, i);
-            if (lane == j) {
-                before = m;
-                after = mn;
+        float f = gt.forget, i = gt.in;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const float fo = __shfl_up(f, off, 64), io = __shfl_up(i, off, 64);
+            if (lane >= off) {
+                i = fmaxf(f + io, i);
+                f += fo;
             }
-            m = mn;
         }
+        const float after = fmaxf(f + m, i), shifted = __shfl_up(after, 1, 64), before = lane ? shifted : m;
         if (lane < n) *(float4 *)(p.gates + (row * d.R + head) * 4) = float4{expf(gt.forget + before - after), expf(gt.in - after), expf(-after), 0.f};
+        m = __shfl(after, n - 1, 64);
     }
     if (lane == 0) *mx = m;
 }
@@ -368,32 +373,28 @@ template <typename T> __global__ __launch_bounds__(256) void delta_prepare_kerne
         if (ch < d.col_v()) buf[ch] = y;
         else p.v[(size_t)row * d.H * d.vp + ch - d.col_v()] = y;
     }
-    float *scal = p.scal + (size_t)row * (d.H + d.G);
-    for (int h = tid; h < d.H; h += 256) scal[h] = sigmoidf(proj[d.col_b() + h]);
+    for (int h = tid; h < d.H; h += 256) p.beta[(size_t)row * d.H + h] = sigmoidf(proj[d.col_b() + h]);
     for (int i = tid; i < d.low(); i += 256) Elem<T>::st((T *)p.low, (size_t)row * d.low() + i, proj[d.col_low() + i]);
     __syncthreads();
     for (int hk = wave; hk < d.G; hk += 4) {
         const float *q = buf + hk * d.dp, *k = buf + d.col_k() + hk * d.dp;
-        float qq = 0.f, kk = 0.f, qk = 0.f;
+        float qq = 0.f, kk = 0.f;
         for (int i = lane; i < d.dp; i += 64) {
             qq = fmaf(q[i], q[i], qq);
             kk = fmaf(k[i], k[i], kk);
-            qk = fmaf(q[i], k[i], qk);
         }
         const float qn = 1.0f / sqrtf((float)d.d) / sqrtf(wave_sum(qq) + 1e-6f), kn = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
-        qk = wave_sum(qk) * qn * kn;
         float *dst = p.qk + (size_t)row * 2 * d.G * d.dp + hk * d.dp;
         for (int i = lane; i < d.dp; i += 64) {
             dst[i] = q[i] * qn;
             dst[d.col_k() + i] = k[i] * kn;
         }
-        if (lane == 0) scal[d.H + hk] = qk;
     }
 }
 int delta_prepare(const DeltaParams &p, int dtype, hipStream_t s) {
     int rc = check_delta(p);
     if (rc) return rc;
-    MYNN_REQUIRE(p.qk && p.v && p.scal && p.low, MYNN_ERR_INVALID, "delta prepare: null operand");
+    MYNN_REQUIRE(p.qk && p.v && p.beta && p.low, MYNN_ERR_INVALID, "delta prepare: null operand");
     const size_t lds = (size_t)p.d.col_v() * 4;
     return dispatch_dense(dtype, [&](auto *t) {
         using T = std::remove_pointer_t<decltype(t)>;
@@ -404,184 +405,341 @@ int delta_prepare(const DeltaParams &p, int dtype, hipStream_t s) {
     });
 }
 
-template <typename T> __global__ __launch_bounds__(256) void delta_decays_kernel(DeltaParams p, size_t total) {
-    const size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
-    if (i >= total) return;
-    const DeltaDims &d = p.d;
-    const int n = d.H * d.dp, c = (int)(i % n);
-    float *at = p.dec + i / n * d.n_low() + c;
-    const float ea = expf(Elem<T>::ld((const T *)p.a_log, c / d.dp));  // (a head's channels come in fours)
-    float4 v = *(const float4 *)at;
-    float *f = (float *)&v;
-#pragma unroll
-    for (int e = 0; e < 4; e++) f[e] = expf(-ea * softplusf(f[e] + Elem<T>::ld((const T *)p.dt_bias, c + e)));
-    *(float4 *)at = v;
+// ---- the recurrence, a block of kBlock tokens at a time -----------------------------------------------------------------
+constexpr int kBlock = 16;
+static_assert(kBlock == kRecurrentBlock, "what the buffers are laid out for");
+// operands of block n of (sequence, head) x: [x * nb + n] of each array
+struct BlockOperands {
+    float *kt, *qt, *kh, *gam, *T, *B;  // [16][KD], [16][KD], [KD][16], [KD], [16][16], [16][16]
+};
+__device__ __host__ inline BlockOperands block_operands(float *base, size_t blocks, int KD, bool delta) {
+    BlockOperands o;
+    o.qt = base;
+    o.kh = o.qt + blocks * kBlock * KD;
+    o.gam = o.kh + blocks * kBlock * KD;
+    o.B = o.gam + blocks * KD;
+    o.T = o.B + blocks * kBlock * kBlock;
+    o.kt = o.T + (delta ? blocks * kBlock * kBlock : 0);
+    return o;
 }
-int delta_decays(const DeltaParams &p, int dtype, hipStream_t s) {
-    MYNN_REQUIRE(p.dec && p.a_log && p.dt_bias, MYNN_ERR_INVALID, "delta decays: null operand");
-    const size_t total = (size_t)p.B * p.S * p.d.H * p.d.dp;
-    return dispatch_dense(dtype, [&](auto *t) {
-        using T = std::remove_pointer_t<decltype(t)>;
-        MYNN_LAUNCH(delta_decays_kernel<T>, dim3((unsigned)((total / 4 + 255) / 256)), dim3(256), 0, s, p, total);
-        return launch_status("delta_decays_kernel");
-    });
+size_t recurrent_block_floats(int B, int S, int H, int dp, bool delta) {
+    const size_t blocks = (size_t)B * H * ((S + kBlock - 1) / kBlock);
+    const int KD = recurrent_keys(dp);
+    return blocks * ((size_t)(delta ? 3 : 2) * kBlock * KD + KD + (delta ? 2 : 1) * kBlock * kBlock);
 }
 
-// ---- the recurrence over tokens -----------------------------------------------------------------------------------------
+// G q (and G k) of every token, the keys carried to the block's end, G of the whole block; thread per key channel.
+// q, k, g in LDS [16][ldl]; carry(t): what a key of token t is multiplied by
+template <bool DELTA, typename Decay, typename Put>
+__device__ inline void block_vectors(const BlockOperands &o, size_t blk, int KD, const float *q, const float *k, int ldl, Decay &&decay, Put &&put) {
+    for (int c = threadIdx.x; c < KD; c += 256) {
+        float G = 1.f;
+#pragma unroll
+        for (int j = 0; j < kBlock; j++) {
+            G *= decay(j, c);
+            o.qt[(blk * kBlock + j) * KD + c] = q[j * ldl + c] * G;
+            if constexpr (DELTA) o.kt[(blk * kBlock + j) * KD + c] = k[j * ldl + c] * G;
+        }
+        o.gam[blk * KD + c] = G;
+        float w[kBlock], R = 1.f;
+#pragma unroll
+        for (int i = kBlock - 1; i >= 0; i--) {
+            w[i] = k[i * ldl + c] * put(i) * R;
+            R *= decay(i, c);
+        }
+#pragma unroll
+        for (int i = 0; i < kBlock; i += 4) *(float4 *)(o.kh + (blk * KD + c) * kBlock + i) = *(const float4 *)(w + i);
+    }
+}
+
+template <typename T, int KT>  // KD = 64 KT
+__global__ __launch_bounds__(256) void delta_blocks_kernel(DeltaParams p, float *base) {
+    constexpr int KD = 64 * KT, LDL = KD + 4;
+    __shared__ __align__(16) float ks[kBlock * LDL], qs[kBlock * LDL], gs[kBlock * LDL];
+    __shared__ float As[kBlock][kBlock + 1], beta[kBlock];
+    const DeltaDims &d = p.d;
+    const int n = blockIdx.x, h = blockIdx.y, b = blockIdx.z, nb = gridDim.x, hk = h / (d.H / d.G), tid = threadIdx.x;
+    const size_t blk = ((size_t)b * d.H + h) * nb + n, row0 = (size_t)b * p.S + n * kBlock;
+    const int live = min(kBlock, p.S - n * kBlock);
+    const BlockOperands o = block_operands(base, (size_t)gridDim.z * d.H * nb, KD, true);
+    const float ea = expf(Elem<T>::ld((const T *)p.a_log, h));
+    for (int i = tid; i < kBlock * KD / 4; i += 256) {
+        const int t = i / (KD / 4), c = i % (KD / 4) * 4;
+        // (tokens past the portion: no key, no query, no decay; channels past the head: nothing)
+        float4 k = float4{0.f, 0.f, 0.f, 0.f}, q = k, g = float4{1.f, 1.f, 1.f, 1.f};
+        if (t < live && c < d.dp) {
+            const float *src = p.qk + (row0 + t) * 2 * d.G * d.dp + hk * d.dp + c;
+            q = *(const float4 *)src;
+            k = *(const float4 *)(src + d.col_k());
+            const float4 a = *(const float4 *)(p.dec + (row0 + t) * d.n_low() + h * d.dp + c);
+            const float f[4] = {a.x, a.y, a.z, a.w};
+            float *gv = (float *)&g;
+#pragma unroll
+            for (int e = 0; e < 4; e++) gv[e] = expf(-ea * softplusf(f[e] + Elem<T>::ld((const T *)p.dt_bias, h * d.dp + c + e)));
+        }
+        *(float4 *)(ks + t * LDL + c) = k;
+        *(float4 *)(qs + t * LDL + c) = q;
+        *(float4 *)(gs + t * LDL + c) = g;
+    }
+    if (tid < kBlock) beta[tid] = tid < live ? p.beta[(row0 + tid) * d.H + h] : 0.f;
+    __syncthreads();
+    // A and B: thread = (earlier token i, sixteenth of the channels)
+    {
+        const int i = tid >> 4, sl = tid & 15;
+        float w[4 * KT];
+        float *Bm = o.B + blk * kBlock * kBlock;
+        float own = 0.f;
+#pragma unroll
+        for (int P = 0; P < KT; P++) {
+            *(float4 *)(w + 4 * P) = *(const float4 *)(ks + i * LDL + P * 64 + sl * 4);
+            const float4 q = *(const float4 *)(qs + i * LDL + P * 64 + sl * 4);
+            own = fmaf(w[4 * P], q.x, fmaf(w[4 * P + 1], q.y, fmaf(w[4 * P + 2], q.z, fmaf(w[4 * P + 3], q.w, own))));
+        }
+        own = group_sum<16>(own);
+        if (sl <= i) Bm[sl * kBlock + i] = sl == i ? own : 0.f;  // (row sl, column i: nothing above the diagonal)
+        for (int j = i + 1; j < kBlock; j++) {
+            float a = 0.f, c = 0.f;
+#pragma unroll
+            for (int P = 0; P < KT; P++) {
+                const float4 g = *(const float4 *)(gs + j * LDL + P * 64 + sl * 4), k = *(const float4 *)(ks + j * LDL + P * 64 + sl * 4);
+                const float4 q = *(const float4 *)(qs + j * LDL + P * 64 + sl * 4);
+                w[4 * P] *= g.x; w[4 * P + 1] *= g.y; w[4 * P + 2] *= g.z; w[4 * P + 3] *= g.w;
+                a = fmaf(w[4 * P], k.x, fmaf(w[4 * P + 1], k.y, fmaf(w[4 * P + 2], k.z, fmaf(w[4 * P + 3], k.w, a))));
+                c = fmaf(w[4 * P], q.x, fmaf(w[4 * P + 1], q.y, fmaf(w[4 * P + 2], q.z, fmaf(w[4 * P + 3], q.w, c))));
+            }
+            a = group_sum<16>(a);
+            c = group_sum<16>(c);
+            if (sl == 0) {
+                As[j][i] = a;
+                Bm[j * kBlock + i] = c;
+            }
+        }
+    }
+    block_vectors<true>(o, blk, KD, qs, ks, LDL, [&](int t, int c) { return gs[t * LDL + c]; }, [](int) { return 1.f; });
+    __syncthreads();
+    // T = (1 + diag(beta) A)^-1 diag(beta), a column per thread
+    if (tid < kBlock) {
+        float x[kBlock];
+#pragma unroll
+        for (int j = 0; j < kBlock; j++) {
+            float s = j == tid ? 1.f : 0.f;
+#pragma unroll
+            for (int i = 0; i < j; i++) s = i >= tid ? fmaf(-As[j][i], x[i], s) : s;
+            x[j] = beta[j] * s;
+            o.T[(blk * kBlock + j) * kBlock + tid] = x[j];
+        }
+    }
+}
+
+template <int KT>
+__global__ __launch_bounds__(256) void memory_blocks_kernel(MemoryParams p, float *base) {
+    constexpr int KD = 64 * KT, LDL = KD + 4;
+    __shared__ __align__(16) float ks[kBlock * LDL], qs[kBlock * LDL];
+    __shared__ float keep[kBlock], put[kBlock];
+    const ParallelDims &d = p.d;
+    const int n = blockIdx.x, h = blockIdx.y, b = blockIdx.z, nb = gridDim.x, tid = threadIdx.x;
+    const size_t blk = ((size_t)b * d.R + h) * nb + n, row0 = (size_t)b * p.S + n * kBlock;
+    const int live = min(kBlock, p.S - n * kBlock);
+    const BlockOperands o = block_operands(base, (size_t)gridDim.z * d.R * nb, KD, false);
+    for (int i = tid; i < kBlock * KD / 4; i += 256) {
+        const int t = i / (KD / 4), c = i % (KD / 4) * 4;
+        float4 k = float4{0.f, 0.f, 0.f, 0.f}, q = k;
+        if (t < live && c < d.rdp) {
+            const float *src = p.proj + (row0 + t) * d.n_in() + h * d.rdp + c;
+            q = *(const float4 *)(src + d.mem_q());
+            k = *(const float4 *)(src + d.mem_k());
+            q.x *= p.q_scale; q.y *= p.q_scale; q.z *= p.q_scale; q.w *= p.q_scale;
+        }
+        *(float4 *)(ks + t * LDL + c) = k;
+        *(float4 *)(qs + t * LDL + c) = q;
+    }
+    if (tid < kBlock) {
+        const float *g = p.gates + ((row0 + min(tid, live - 1)) * d.R + h) * 4;
+        keep[tid] = tid < live ? g[0] : 1.f;
+        put[tid] = tid < live ? g[1] : 0.f;
+    }
+    __syncthreads();
+    {
+        const int j = tid >> 4, i = tid & 15;
+        float a = 0.f;
+#pragma unroll 8
+        for (int c = 0; c < KD; c += 4) {
+            const float4 q = *(const float4 *)(qs + j * LDL + c), k = *(const float4 *)(ks + i * LDL + c);
+            a = fmaf(q.x, k.x, fmaf(q.y, k.y, fmaf(q.z, k.z, fmaf(q.w, k.w, a))));
+        }
+        a = i <= j ? a * put[i] : 0.f;
+        for (int t = i + 1; t <= j; t++) a *= keep[t];
+        o.B[(blk * kBlock + j) * kBlock + i] = a;
+    }
+    block_vectors<false>(o, blk, KD, qs, ks, LDL, [&](int t, int) { return keep[t]; }, [&](int t) { return put[t]; });
+}
+
 struct RecurrenceParams {
-    int S, H, group, dp, ncol, nv;       // group: heads per key head; ncol: state columns, the first nv of them have a value (else 1)
-    const float *q, *k, *v, *g;          // row 0 of each; heads at dp / dp / vp / dp
-    long ldq, ldk, ldv, ldg;
+    int S, H, dp, ncol, nv;              // ncol: state columns, the first nv of them have a value (else 1)
+    const float *v;                      // row * ldv + h * vp + column
+    long ldv;
     int vp;
-    float q_scale;
-    const float *scal;                   // delta: [row][H + G]; memory: [row][H][4]
+    float *base;                         // block operands
     float *state;
     long state_stride;
     float *o;                            // [row][H][op]
     int op;
     const int32_t *d_past;
 };
-constexpr int kRecThreads = 256, kRecWaves = 4;
 
-template <bool DELTA, int LC, int RP>
-__global__ __launch_bounds__(kRecThreads) void recurrence_kernel(RecurrenceParams p) {
-    constexpr int KD = LC * RP, CPW = kRecWaves * 64 / LC, TC = KD <= 32 ? 8 : KD <= 128 ? 16 : KD <= 256 ? 8 : 4, NA = DELTA ? 3 : 2;
-    constexpr int NL = (TC * KD / 4 + kRecThreads - 1) / kRecThreads;
-    constexpr int NV = (TC * CPW + kRecThreads - 1) / kRecThreads;
-    static_assert(TC <= LC && TC <= 64, "a lane per token keeps its output");
-    extern __shared__ __align__(16) float sm[];  // [2][NA][TC][KD], [2][TC][CPW], [2][TC][2]
-    float *vals = sm + 2 * NA * TC * KD, *sc = vals + 2 * TC * CPW;
-    const int h = blockIdx.x, c0 = blockIdx.y * CPW, b = blockIdx.z, hk = h / p.group, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int r = lane % LC, cg = wave * (64 / LC) + lane / LC, col = c0 + cg, q4 = p.dp / 4;
-    const size_t row0 = (size_t)b * p.S;
+// Sixteen state columns of a head per workgroup; wave w holds key channels 16 TW w .. of them as TW accumulator tiles of
+// v_mfma_f32_16x16x4_f32 (lane (quad, c): channels 4 quad .. + 3 of a tile, column c).  An accumulator register is at the
+// same time the second operand of the next product, over the four channels 4 quad + i.
+template <bool DELTA, int TW>
+__global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
+    constexpr int KD = 64 * TW;
+    __shared__ __align__(16) float4 part[2][4][2][64];
+    typedef float f4_t __attribute__((ext_vector_type(4)));
+    const int h = blockIdx.x, c0 = blockIdx.y * 16, b = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c16 = lane & 15, quad = lane >> 4;
+    const int nb = (p.S + kBlock - 1) / kBlock, col = c0 + c16, k0 = wave * 16 * TW;
+    const BlockOperands op = block_operands(p.base, (size_t)gridDim.z * p.H * nb, KD, DELTA);
+    const size_t blk0 = ((size_t)b * p.H + h) * nb, row0 = (size_t)b * p.S;
     float *at = p.state + (size_t)b * p.state_stride + ((size_t)h * p.ncol + min(col, p.ncol - 1)) * p.dp;
-    Column<LC, RP> S;
-    S.load(at, r, p.dp);
-    const float *src[3] = {p.q + row0 * p.ldq + hk * p.dp, p.k + row0 * p.ldk + hk * p.dp, DELTA ? p.g + row0 * p.ldg + h * p.dp : nullptr};
-    const long ld[3] = {p.ldq, p.ldk, p.ldg};
-    int lt[NL], lc4[NL];
+    const bool fresh = *p.d_past == 0;
+    f4_t S[TW];
 #pragma unroll
-    for (int i = 0; i < NL; i++) {
-        const int idx = tid + i * kRecThreads;
-        lt[i] = idx / q4;
-        lc4[i] = idx % q4 * 4;
+    for (int t = 0; t < TW; t++) {
+        const int c = k0 + 16 * t + 4 * quad;
+        S[t] = f4_t{0.f, 0.f, 0.f, 0.f};
+        if (!fresh && c < p.dp) S[t] = *(const f4_t *)(at + c);
     }
-    float4 pre[NA][NL];
-    float pv[NV], ps[2];
-    auto request = [&](int t0) {
+    struct Block {
+        f4_t qt[TW], kt[DELTA ? TW : 1], kh[TW], gam[TW], B, T;
+        float v[4];
+    };
+    auto request = [&](Block &x, int n) {
+        const size_t blk = blk0 + min(n, nb - 1);
 #pragma unroll
-        for (int i = 0; i < NL; i++)
-            if (lt[i] < TC) {
-                const int t = min(t0 + lt[i], p.S - 1);
-#pragma unroll
-                for (int a = 0; a < NA; a++) pre[a][i] = *(const float4 *)(src[a] + (size_t)t * ld[a] + lc4[i]);
-            }
-#pragma unroll
-        for (int i = 0; i < NV; i++) {
-            const int idx = tid + i * kRecThreads, t = min(t0 + idx / CPW, p.S - 1), c = c0 + idx % CPW;
-            pv[i] = 1.f;
-            if (idx < TC * CPW && c < p.nv) pv[i] = p.v[(row0 + t) * p.ldv + h * p.vp + c];
+        for (int t = 0; t < TW; t++) {
+            const int c = k0 + 16 * t;
+            x.qt[t] = *(const f4_t *)(op.qt + (blk * kBlock + c16) * KD + c + 4 * quad);
+            if constexpr (DELTA) x.kt[t] = *(const f4_t *)(op.kt + (blk * kBlock + c16) * KD + c + 4 * quad);
+            x.kh[t] = *(const f4_t *)(op.kh + (blk * KD + c + c16) * kBlock + 4 * quad);
+            x.gam[t] = *(const f4_t *)(op.gam + blk * KD + c + 4 * quad);
         }
-        if (tid < TC) {
-            const size_t row = row0 + min(t0 + tid, p.S - 1);
-            if constexpr (DELTA) {
-                const int G = p.H / p.group;
-                ps[0] = p.scal[row * (p.H + G) + h];
-                ps[1] = p.scal[row * (p.H + G) + p.H + hk];
-            } else {
-                ps[0] = p.scal[(row * p.H + h) * 4];
-                ps[1] = p.scal[(row * p.H + h) * 4 + 1];
-            }
+        x.B = *(const f4_t *)(op.B + (blk * kBlock + c16) * kBlock + 4 * quad);
+        if constexpr (DELTA) x.T = *(const f4_t *)(op.T + (blk * kBlock + c16) * kBlock + 4 * quad);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int t = min(min(n, nb - 1) * kBlock + 4 * quad + i, p.S - 1);
+            x.v[i] = col < p.nv ? p.v[(row0 + t) * p.ldv + h * p.vp + col] : 1.f;
         }
     };
-    request(0);
-    for (int i = tid; i < 2 * NA * TC * KD; i += kRecThreads) sm[i] = 0.f;  // (channels past dp stay zero)
-    S.clear(*p.d_past == 0, r, p.dp);
-    __syncthreads();
-    for (int t0 = 0, buf = 0; t0 < p.S; t0 += TC, buf ^= 1) {
-        float *x = sm + buf * NA * TC * KD, *vb = vals + buf * TC * CPW, *sb = sc + buf * TC * 2;
+    auto step = [&](const Block &x, int n) {
+        f4_t pq = {0.f, 0.f, 0.f, 0.f}, pk = pq;
 #pragma unroll
-        for (int i = 0; i < NL; i++)
-            if (lt[i] < TC)
+        for (int t = 0; t < TW; t++)
 #pragma unroll
-                for (int a = 0; a < NA; a++) *(float4 *)(x + (a * TC + lt[i]) * KD + lc4[i]) = pre[a][i];
-#pragma unroll
-        for (int i = 0; i < NV; i++)
-            if (tid + i * kRecThreads < TC * CPW) vb[tid + i * kRecThreads] = pv[i];
-        if (tid < TC) {
-            sb[2 * tid] = ps[0];
-            sb[2 * tid + 1] = ps[1];
-        }
-        __syncthreads();  // (the other buffer was read before the barrier of the chunk before)
-        if (t0 + TC < p.S) request(t0 + TC);
-        float mine = 0.f;
-        const int n = min(TC, p.S - t0);
-        for (int t = 0; t < n; t++) {
-            float q[RP], k[RP], g[RP];
-            channels_of<LC, RP>(x + t * KD, r, q);
-            channels_of<LC, RP>(x + (TC + t) * KD, r, k);
-            const float s0 = sb[2 * t], s1 = sb[2 * t + 1], v = vb[t * CPW + cg];
-            float o = 0.f;
-            if constexpr (DELTA) {
-                channels_of<LC, RP>(x + (2 * TC + t) * KD, r, g);
-                float a = 0.f;
-#pragma unroll
-                for (int j = 0; j < RP; j++) {
-                    S.s[j] *= g[j];
-                    a = fmaf(S.s[j], k[j], a);
-                    o = fmaf(S.s[j], q[j], o);
-                }
-                a = group_sum<LC>(a);
-                o = group_sum<LC>(o);
-                const float u = s0 * (v - a);
-#pragma unroll
-                for (int j = 0; j < RP; j++) S.s[j] = fmaf(k[j], u, S.s[j]);
-                o = fmaf(s1, u, o);  // (s1 = q . k: the read-out sees this token's write)
-            } else {
-                const float pvv = s1 * v;
-#pragma unroll
-                for (int j = 0; j < RP; j++) {
-                    S.s[j] = fmaf(k[j], pvv, s0 * S.s[j]);
-                    o = fmaf(S.s[j], q[j], o);
-                }
-                o = group_sum<LC>(o) * p.q_scale;
+            for (int i = 0; i < 4; i++) {
+                pq = __builtin_amdgcn_mfma_f32_16x16x4f32(x.qt[t][i], S[t][i], pq, 0, 0, 0);
+                if constexpr (DELTA) pk = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kt[t][i], S[t][i], pk, 0, 0, 0);
             }
-            mine = r == t ? o : mine;
+        float4(*my)[64] = part[n & 1][wave];
+        my[0][lane] = __builtin_bit_cast(float4, pq);
+        if constexpr (DELTA) my[1][lane] = __builtin_bit_cast(float4, pk);
+#pragma unroll
+        for (int t = 0; t < TW; t++) S[t] *= x.gam[t];
+        __syncthreads();  // (the other half of `part` was read before the barrier of the block before)
+        f4_t u;
+        if constexpr (DELTA) {
+            f4_t r = {x.v[0], x.v[1], x.v[2], x.v[3]};
+#pragma unroll
+            for (int w = 0; w < 4; w++) r -= __builtin_bit_cast(f4_t, part[n & 1][w][1][lane]);
+            u = f4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int i = 0; i < 4; i++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(x.T[i], r[i], u, 0, 0, 0);
+        } else u = f4_t{x.v[0], x.v[1], x.v[2], x.v[3]};
+#pragma unroll
+        for (int t = 0; t < TW; t++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kh[t][i], u[i], S[t], 0, 0, 0);
+        if (wave == (n & 3)) {
+            f4_t out = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int w = 0; w < 4; w++) out += __builtin_bit_cast(f4_t, part[n & 1][w][0][lane]);
+#pragma unroll
+            for (int i = 0; i < 4; i++) out = __builtin_amdgcn_mfma_f32_16x16x4f32(x.B[i], u[i], out, 0, 0, 0);
+            if (col < p.ncol)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const int t = n * kBlock + 4 * quad + i;
+                    if (t < p.S) p.o[((row0 + t) * p.H + h) * p.op + col] = out[i];
+                }
         }
-        if (r < n && col < p.ncol) p.o[((row0 + t0 + r) * p.H + h) * p.op + col] = mine;
+    };
+    Block x, y;
+    request(x, 0);
+    for (int n = 0; n < nb; n += 2) {
+        request(y, n + 1);
+        step(x, n);
+        if (n + 1 >= nb) break;
+        request(x, n + 2);
+        step(y, n + 1);
     }
-    if (col < p.ncol) S.store(at, r, p.dp);
+    if (col < p.ncol)
+#pragma unroll
+        for (int t = 0; t < TW; t++) {
+            const int c = k0 + 16 * t + 4 * quad;
+            if (c < p.dp) *(f4_t *)(at + c) = S[t];
+        }
 }
 
+// f(KT): KD = 64 KT key channels
+template <typename F> static int dispatch_keys(int dp, F &&f) {
+    using std::integral_constant;
+    switch (recurrent_keys(dp)) {
+    case 64: return f(integral_constant<int, 1>{});
+    case 128: return f(integral_constant<int, 2>{});
+    case 256: return f(integral_constant<int, 4>{});
+    default: return f(integral_constant<int, 8>{});
+    }
+}
 template <bool DELTA> static int launch_recurrence(const RecurrenceParams &p, int B, hipStream_t s) {
-    MYNN_REQUIRE(p.q && p.k && p.v && p.scal && p.state && p.o && p.d_past && (!DELTA || p.g) && B <= 65535, MYNN_ERR_INVALID, "recurrence: bad operand");
-    return dispatch_columns(p.dp, [&](auto lc, auto rp) {
-        constexpr int LC = decltype(lc)::value, RP = decltype(rp)::value, KD = LC * RP, CPW = kRecWaves * 64 / LC;
-        constexpr int TC = KD <= 32 ? 8 : KD <= 128 ? 16 : KD <= 256 ? 8 : 4, NA = DELTA ? 3 : 2;
-        auto kernel = recurrence_kernel<DELTA, LC, RP>;
-        const size_t lds = (size_t)(2 * NA * TC * KD + 2 * TC * CPW + 4 * TC) * 4;
-        int rc = raise_lds(kernel, lds);
-        if (rc) return rc;
-        MYNN_LAUNCH(kernel, dim3(p.H, (p.ncol + CPW - 1) / CPW, B), dim3(kRecThreads), lds, s, p);
+    MYNN_REQUIRE(p.v && p.base && p.state && p.o && p.d_past && B <= 65535 && recurrent_dim_supported(p.dp), MYNN_ERR_INVALID, "recurrence: bad operand");
+    return dispatch_keys(p.dp, [&](auto kt) {
+        constexpr int KT = decltype(kt)::value;
+        MYNN_LAUNCH((recurrence_kernel<DELTA, KT>), dim3(p.H, (p.ncol + 15) / 16, B), dim3(256), 0, s, p);
         return launch_status("recurrence_kernel");
+    });
+}
+int delta_blocks(const DeltaParams &p, int dtype, hipStream_t s) {
+    int rc = check_delta(p);
+    if (rc) return rc;
+    MYNN_REQUIRE(p.qk && p.dec && p.beta && p.blocks && p.a_log && p.dt_bias && p.d.H <= 65535 && p.B <= 65535, MYNN_ERR_INVALID, "delta blocks: bad operand");
+    return dispatch_dense(dtype, [&](auto *t) {
+        using T = std::remove_pointer_t<decltype(t)>;
+        return dispatch_keys(p.d.dp, [&](auto kt) {
+            constexpr int KT = decltype(kt)::value;
+            MYNN_LAUNCH((delta_blocks_kernel<T, KT>), dim3((p.S + kBlock - 1) / kBlock, p.d.H, p.B), dim3(256), 0, s, p, p.blocks);
+            return launch_status("delta_blocks_kernel");
+        });
     });
 }
 int delta_recurrence(const DeltaParams &p, hipStream_t s) {
     const DeltaDims &d = p.d;
     RecurrenceParams r{};
-    r.S = p.S; r.H = d.H; r.group = d.H / d.G; r.dp = d.dp; r.ncol = r.nv = d.v;
-    r.q = p.qk; r.k = p.qk + d.col_k(); r.v = p.v; r.g = p.dec;
-    r.ldq = r.ldk = 2 * d.G * d.dp; r.ldv = d.H * d.vp; r.ldg = d.n_low();
-    r.vp = d.vp; r.q_scale = 1.f; r.scal = p.scal; r.state = p.state; r.state_stride = p.state_stride; r.o = p.o; r.op = d.vp; r.d_past = p.d_past;
+    r.S = p.S; r.H = d.H; r.dp = d.dp; r.ncol = r.nv = d.v; r.v = p.v; r.ldv = d.H * d.vp; r.vp = d.vp; r.base = p.blocks;
+    r.state = p.state; r.state_stride = p.state_stride; r.o = p.o; r.op = d.vp; r.d_past = p.d_past;
     return launch_recurrence<true>(r, p.B, s);
+}
+int memory_blocks(const MemoryParams &p, hipStream_t s) {
+    MYNN_REQUIRE(p.proj && p.gates && p.blocks && p.S > 0 && p.d.R <= 65535 && p.B <= 65535 && recurrent_dim_supported(p.d.rdp), MYNN_ERR_INVALID, "memory blocks: bad operand");
+    return dispatch_keys(p.d.rdp, [&](auto kt) {
+        constexpr int KT = decltype(kt)::value;
+        MYNN_LAUNCH(memory_blocks_kernel<KT>, dim3((p.S + kBlock - 1) / kBlock, p.d.R, p.B), dim3(256), 0, s, p, p.blocks);
+        return launch_status("memory_blocks_kernel");
+    });
 }
 int memory_recurrence(const MemoryParams &p, hipStream_t s) {
     const ParallelDims &d = p.d;
     RecurrenceParams r{};
-    r.S = p.S; r.H = d.R; r.group = 1; r.dp = d.rdp; r.ncol = d.rv + 1; r.nv = d.rv;
-    r.q = p.proj + d.mem_q(); r.k = p.proj + d.mem_k(); r.v = p.proj + d.mem_v();
-    r.ldq = r.ldk = r.ldv = d.n_in(); r.vp = d.rvp; r.q_scale = p.q_scale; r.scal = p.gates; r.state = p.state; r.state_stride = p.state_stride;
-    r.o = p.o; r.op = pad_to(d.rv + 1, 4); r.d_past = p.d_past;
+    r.S = p.S; r.H = d.R; r.dp = d.rdp; r.ncol = d.rv + 1; r.nv = d.rv; r.v = p.proj + d.mem_v(); r.ldv = d.n_in(); r.vp = d.rvp; r.base = p.blocks;
+    r.state = p.state; r.state_stride = p.state_stride; r.o = p.o; r.op = pad_to(d.rv + 1, 4); r.d_past = p.d_past;
     return launch_recurrence<false>(r, p.B, s);
 }
 
