@@ -459,7 +459,7 @@ __global__ __launch_bounds__(256) void gemm_nt_f32_kernel(float *out, const floa
     const int m0 = blockIdx.y * 128, n0 = blockIdx.x * 64;
     const int lr = tid >> 2, lc = (tid & 3) * 4;
     if constexpr (GROUPED) {
-        const int grp = gr.tile_group[blockIdx.y];
+        const int grp = gr.tile_group[blockIdx.y * 128 / gr.group_rows];
         if (grp < 0) return;
         B += (size_t)grp * gr.group_elems;
     }
@@ -542,8 +542,9 @@ int gemm_grouped(void *out, const void *act, const void *wt, const GroupedRows &
     MYNN_REQUIRE(g.gather == (epi == GEMM_SILU) && (epi != GEMM_SILU || (N % 64 == 0 && g.scale)), MYNN_ERR_INVALID, "grouped gemm: store %d of N=%d", epi, N);
     if (dtype == MYNN_BF16) return gemm_grouped_bf16(out, act, wt, g, N, K, epi, s);
     MYNN_REQUIRE(dtype == MYNN_F32, MYNN_ERR_UNSUPPORTED, "grouped gemm: dtype %d", dtype);
-    static_assert(kGroupRows == 128, "the f32 kernel's row tile");
-    const dim3 grid((N + 63) / 64, g.tiles);
+    MYNN_REQUIRE(g.group_rows % 128 == 0, MYNN_ERR_INVALID, "grouped gemm: groups of %d rows", g.group_rows);
+    const dim3 grid((N + 63) / 64, g.tiles * (g.group_rows / 128));
+    MYNN_REQUIRE(grid.y <= 65535, MYNN_ERR_UNSUPPORTED, "grouped gemm: %d tiles", g.tiles);
     if (epi == GEMM_SILU)
         MYNN_LAUNCH((gemm_nt_f32_kernel<DENSE_GEGLU, true>), grid, dim3(256), 0, s, (float *)out, (const float *)act, (const float *)wt, 0, N, K, nullptr, g);
     else

@@ -21,14 +21,16 @@ struct ExpertParams {
     float *score;             // [rows, top]
     // (assignment = row * top + i) sorted by expert, every expert's share padded to whole tiles
     int32_t *tile_expert;     // [max_tiles], -1: not used
-    int32_t *slot;            // [max_tiles * kGroupRows] assignment, -1: padding
-    void *hsort;              // T [max_tiles * kGroupRows, fp]
+    int32_t *slot;            // [max_tiles * rows of a tile] assignment, -1: padding
+    void *hsort;              // T [max_tiles * rows of a tile, fp]
     float *parts;             // f32 [rows * top, ld] (top > 1)
     void *y;                  // T [rows, ld]
 };
-inline int expert_tiles(int rows, int E, int top) {
+// rows of a tile: large ones once the experts have enough rows to fill them; tiles that any split of the rows needs
+inline int expert_group_rows(int rows, int E, int top) { return (long)rows * top >= 192L * E ? 256 : 128; }
+inline int expert_tiles(int rows, int E, int top, int group_rows) {
     const long a = (long)rows * top;
-    return (int)(a / kGroupRows + (a < E ? a : E));
+    return (int)(a / group_rows + (a < E ? a : E));
 }
 // one row: y = the experts' sum; x and the router's logits are there
 int expert_gateup_row(const ExpertParams &p, int dtype, hipStream_t s);

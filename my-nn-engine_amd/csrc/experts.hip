@@ -3,7 +3,7 @@
 // One row (decode): the router's logits come from the ordinary one-row linear; expert_gateup_row_kernel picks its expert from
 // them (every workgroup for itself) and streams that expert's rows, expert_down_row_kernel adds the experts' products up in
 // f32.  Several rows: route_rows_kernel scores a few rows per workgroup, sort_kernel lists the assignments expert by expert in
-// whole tiles of kGroupRows, and the two products run as grouped matrix-core products over that list (gemm_grouped).
+// whole tiles, and the two products run as grouped matrix-core products over that list (gemm_grouped).
 #include <algorithm>
 
 #include "dense_load.h"
@@ -254,21 +254,21 @@ int expert_route(const ExpertParams &p, int dtype, hipStream_t s) {
 
 // One workgroup: counts per expert, whole tiles per expert, then every assignment takes a place of its expert's.
 constexpr int kSortT = 1024;
-__global__ __launch_bounds__(kSortT) void sort_kernel(const int32_t *choice, int n, int E, int max_tiles, int32_t *tile_expert, int32_t *slot) {
+__global__ __launch_bounds__(kSortT) void sort_kernel(const int32_t *choice, int n, int E, int group_rows, int max_tiles, int32_t *tile_expert, int32_t *slot) {
     extern __shared__ int32_t cnt[];  // [E] counts, then next places
     const int tid = threadIdx.x;
     for (int e = tid; e < E; e += kSortT) cnt[e] = 0;
     for (int i = tid; i < max_tiles; i += kSortT) tile_expert[i] = -1;
-    for (int i = tid; i < max_tiles * kGroupRows; i += kSortT) slot[i] = -1;
+    for (int i = tid; i < max_tiles * group_rows; i += kSortT) slot[i] = -1;
     __syncthreads();
     for (int i = tid; i < n; i += kSortT) atomicAdd(&cnt[choice[i]], 1);
     __syncthreads();
     if (tid == 0) {
         int tile = 0;
         for (int e = 0; e < E; e++) {
-            const int first = tile, tiles = (cnt[e] + kGroupRows - 1) / kGroupRows;
+            const int first = tile, tiles = (cnt[e] + group_rows - 1) / group_rows;
             for (int t = 0; t < tiles; t++) tile_expert[tile++] = e;
-            cnt[e] = first * kGroupRows;
+            cnt[e] = first * group_rows;
         }
     }
     __syncthreads();
@@ -276,7 +276,8 @@ __global__ __launch_bounds__(kSortT) void sort_kernel(const int32_t *choice, int
 }
 int expert_sort(const ExpertParams &p, hipStream_t s) {
     MYNN_REQUIRE(p.choice && p.tile_expert && p.slot && p.rows > 0, MYNN_ERR_INVALID, "experts: null operand");
-    MYNN_LAUNCH(sort_kernel, dim3(1), dim3(kSortT), (size_t)p.E * 4, s, p.choice, p.rows * p.top, p.E, expert_tiles(p.rows, p.E, p.top), p.tile_expert, p.slot);
+    const int gr = expert_group_rows(p.rows, p.E, p.top);
+    MYNN_LAUNCH(sort_kernel, dim3(1), dim3(kSortT), (size_t)p.E * 4, s, p.choice, p.rows * p.top, p.E, gr, expert_tiles(p.rows, p.E, p.top, gr), p.tile_expert, p.slot);
     return launch_status("sort_kernel");
 }
 
@@ -284,14 +285,16 @@ int expert_gateup(const ExpertParams &p, int dtype, hipStream_t s) {
     int rc = check_experts(p);
     if (rc) return rc;
     MYNN_REQUIRE(p.act && p.hsort && p.score && p.slot && p.tile_expert, MYNN_ERR_INVALID, "experts: null operand");
-    GroupedRows g{p.tile_expert, p.slot, p.score, p.top, true, expert_tiles(p.rows, p.E, p.top), (size_t)2 * p.fp * p.ld};
+    const int gr = expert_group_rows(p.rows, p.E, p.top);
+    GroupedRows g{p.tile_expert, p.slot, p.score, p.top, true, expert_tiles(p.rows, p.E, p.top, gr), gr, (size_t)2 * p.fp * p.ld};
     return gemm_grouped(p.hsort, p.act, p.gu, g, 2 * p.fp, p.ld, GEMM_SILU, dtype, s);
 }
 int expert_down(const ExpertParams &p, int dtype, hipStream_t s) {
     int rc = check_experts(p);
     if (rc) return rc;
     MYNN_REQUIRE(p.hsort && p.y && p.slot && p.tile_expert && (p.top == 1 || p.parts), MYNN_ERR_INVALID, "experts: null operand");
-    GroupedRows g{p.tile_expert, p.slot, nullptr, p.top, false, expert_tiles(p.rows, p.E, p.top), (size_t)p.ld * p.fp};
+    const int gr = expert_group_rows(p.rows, p.E, p.top);
+    GroupedRows g{p.tile_expert, p.slot, nullptr, p.top, false, expert_tiles(p.rows, p.E, p.top, gr), gr, (size_t)p.ld * p.fp};
     return gemm_grouped(p.top == 1 ? p.y : (void *)p.parts, p.hsort, p.down, g, p.ld, p.fp, p.top == 1 ? GEMM_PLAIN : GEMM_F32, dtype, s);
 }
 

@@ -336,7 +336,6 @@ __device__ __forceinline__ void gemm_dma_body(T *C, const void *A_, const void *
     tile_of(blockIdx.x, gridDim.x, tiles_m, tiles_n, tm, tn);
     const int m0 = tm * BM, n0 = tn * BN;
     if constexpr (GROUPED) {
-        static_assert(BM == kGroupRows, "a row tile is one group's");
         const int grp = gr.tile_group[tm];
         if (grp < 0) return;
         B += (size_t)grp * gr.group_elems * EB;
@@ -433,7 +432,20 @@ __device__ __forceinline__ void gemm_dma_body(T *C, const void *A_, const void *
     asm volatile("" ::: "memory");
     read_frags(lds, 0, fa[0], fb[0]);
     __builtin_amdgcn_sched_barrier(0);
-    for (int kt = 0; kt < nk; kt++) {
+    int kt0 = 0;
+    if constexpr (GROUPED) {
+        // (a group's rows fill its tiles from the front) a wave whose rows are all padding only brings operands in
+        if (__builtin_amdgcn_readfirstlane(gr.slot[m0 + wrow]) < 0) {
+            for (; kt0 < nk; kt0++) {
+                __builtin_amdgcn_s_waitcnt(0x0070);
+                asm volatile("" ::: "memory");
+                __builtin_amdgcn_s_barrier();
+                asm volatile("" ::: "memory");
+                issue(min(kt0 + 2, nk - 1), kt0 & 1);
+            }
+        }
+    }
+    for (int kt = kt0; kt < nk; kt++) {
         const uint16_t *st = lds + (kt & 1) * kDmaStage, *nx = lds + ((kt + 1) & 1) * kDmaStage;
 #pragma unroll
         for (int ks = 0; ks + 1 < KS; ks++) {
@@ -539,7 +551,7 @@ __global__ __launch_bounds__(G::THREADS) void gemm_nt_dma_kernel(T *C, const voi
                                                                  int32_t *acc_out) {
     gemm_dma_body<T, G, EPI, I8, false>(C, A_, B_, R, M, N, K, Kp, a_scale, b_scale, acc_out, GroupedRows{});
 }
-using TileGroup = GemmTile<kGroupRows, 256, 2, 4>;  // 64 x 64 per wave
+using TileGroup = GemmTile<128, 256, 2, 4>;  // 64 x 64 per wave; groups of many rows: TileDma
 template <typename T, typename G, int EPI>
 __global__ __launch_bounds__(G::THREADS) void gemm_nt_grouped_kernel(T *C, const void *A, const void *B, int N, int K, GroupedRows gr) {
     gemm_dma_body<T, G, EPI, false, true>(C, A, B, nullptr, gr.tiles * G::BM, N, K, K, nullptr, nullptr, nullptr, gr);
@@ -606,16 +618,21 @@ static int gemm_launch_dma(void *out, const void *act, const void *wt, const voi
 
 int gemm_grouped_bf16(void *out, const void *act, const void *wt, const GroupedRows &g, int N, int K, int epi, hipStream_t s) {
     MYNN_REQUIRE(K % 64 == 0 && N % 4 == 0 && aligned16(act) && aligned16(wt), MYNN_ERR_INVALID, "grouped gemm: N=%d K=%d", N, K);
-    auto go = [&](auto kernel) {
-        constexpr size_t lds = dma_lds_bytes<TileGroup>();
+    MYNN_REQUIRE(g.group_rows == TileGroup::BM || g.group_rows == TileDma::BM, MYNN_ERR_INVALID, "grouped gemm: groups of %d rows", g.group_rows);
+    auto launch = [&](auto kernel, size_t lds, int bn, int threads) {
         MYNN_HIP(hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-        MYNN_LAUNCH(kernel, dim3(g.tiles * ((N + TileGroup::BN - 1) / TileGroup::BN)), dim3(TileGroup::THREADS), lds, s, (bf16_t *)out, act, wt, N, K, g);
+        MYNN_LAUNCH(kernel, dim3(g.tiles * ((N + bn - 1) / bn)), dim3(threads), lds, s, (bf16_t *)out, act, wt, N, K, g);
         return launch_status("gemm_nt_grouped_kernel");
     };
-    if (epi == GEMM_SILU) return go(gemm_nt_grouped_kernel<bf16_t, TileGroup, GEMM_SILU>);
-    if (epi == GEMM_F32) return go(gemm_nt_grouped_kernel<bf16_t, TileGroup, GEMM_F32>);
+    auto go = [&](auto e) {
+        constexpr int EPI = decltype(e)::value;
+        if (g.group_rows == TileDma::BM) return launch(gemm_nt_grouped_kernel<bf16_t, TileDma, EPI>, dma_lds_bytes<TileDma>(), TileDma::BN, TileDma::THREADS);
+        return launch(gemm_nt_grouped_kernel<bf16_t, TileGroup, EPI>, dma_lds_bytes<TileGroup>(), TileGroup::BN, TileGroup::THREADS);
+    };
+    if (epi == GEMM_SILU) return go(std::integral_constant<int, GEMM_SILU>{});
+    if (epi == GEMM_F32) return go(std::integral_constant<int, GEMM_F32>{});
     MYNN_REQUIRE(epi == GEMM_PLAIN, MYNN_ERR_UNSUPPORTED, "grouped gemm: store %d", epi);
-    return go(gemm_nt_grouped_kernel<bf16_t, TileGroup, GEMM_PLAIN>);
+    return go(std::integral_constant<int, GEMM_PLAIN>{});
 }
 
 // QuantizedMatMul on the matrix cores for a grid of at least one round of 256-row tiles: K % 128 == 0.

@@ -61,19 +61,18 @@ int dequant_gemm_skinny(void *out, const void *act, const int8_t *wq, bool packe
 // gemm_nt_mfma multiplies by it: out = store(act . wt^T) with the store one of GEMM_*.
 // GEMM_GEGLU, GEMM_F32: bf16 operands (store forms of executors with a 32-bit residual stream; see gemm.hip).
 enum { GEMM_PLAIN = 0, GEMM_RESIDUAL = 1, GEMM_SWIGLU = 2, GEMM_GEGLU = 3, GEMM_F32 = 4, GEMM_SILU = 5 };
-// Grouped product: tiles of kGroupRows rows, each against the weight of its own group.  Place i of the list stands for
+// Grouped product: tiles of group_rows (128 or 256) rows, each against the weight of its own group.  Place i of the list stands for
 // assignment slot[i] (-1: none), which belongs to activation row slot[i] / per_row.
 //   gather: A's row of place i is row slot[i] / per_row, output row i, the sum times scale[slot[i]] (GEMM_SILU: gate and up
 //     rows interleaved in groups of 32, silu(gate) * up of the scaled sums)
 //   else:   A's row is row i, output row slot[i] (GEMM_PLAIN: T, GEMM_F32: f32)
-constexpr int kGroupRows = 128;
 struct GroupedRows {
     const int32_t *tile_group;  // [tiles], -1: nothing to do
-    const int32_t *slot;        // [tiles * kGroupRows]
+    const int32_t *slot;        // [tiles * group_rows]
     const float *scale;
     int per_row;
     bool gather;
-    int tiles;
+    int tiles, group_rows;
     size_t group_elems;         // weight elements per group
 };
 // wt: [groups][N, K], K a multiple of 64; bf16 or f32 (dense.hip)

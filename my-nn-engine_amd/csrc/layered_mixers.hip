@@ -130,12 +130,14 @@ void scratch_experts(MixerScratch &x, const MlpSpec &mlp, const mynn_model_confi
     grow(x.router, (size_t)mlp.experts * 4);
     grow(x.hmid, mlp.top * fp * eb);
     grow(x.chosen, (size_t)mlp.top * 4);
-    const size_t tiles = expert_tiles((int)rows, mlp.experts, mlp.top);
+    // (shorter portions may take the smaller tiles: more of them, fewer rows)
+    const int gr = expert_group_rows((int)rows, mlp.experts, mlp.top);
+    const size_t tiles = expert_tiles((int)rows, mlp.experts, mlp.top, 128), slots = (size_t)gr * expert_tiles((int)rows, mlp.experts, mlp.top, gr);
     grow(x.choice, a * 4);
     grow(x.score, a * 4);
     grow(x.tile_group, tiles * 4);
-    grow(x.slot, tiles * kGroupRows * 4);
-    grow(x.hsort, tiles * kGroupRows * fp * eb);
+    grow(x.slot, slots * 4);
+    grow(x.hsort, slots * fp * eb);
     if (mlp.top > 1) grow(x.parts, a * ld * 4);
 }
 

@@ -20,7 +20,7 @@
 namespace mynn {
 
 __device__ inline float softplusf(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
-__device__ inline float siluf(float x) { return x * sigmoidf(x); }
+__device__ inline float4 silu4(const float4 &x) { return float4{x.x * sigmoidf(x.x), x.y * sigmoidf(x.y), x.z * sigmoidf(x.z), x.w * sigmoidf(x.w)}; }
 
 // f(LC, RP): lanes per column and key channels per lane
 template <typename F> static int dispatch_columns(int dp, F &&f) {
@@ -95,18 +95,17 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(DeltaParams p)
     for (int i = tid; i < KD; i += kStepThreads) gs[i] = 0.f;
     for (int i = tid; i < d.low(); i += kStepThreads) low[i] = proj[d.col_low() + i];
     const bool keeps = h % (d.H / d.G) == 0;  // (the heads of a group share q and k; one of them stores the ring)
-    for (int i = tid; i < 2 * KD + d.vp; i += kStepThreads) {
+    for (int i = tid * 4; i < 2 * KD + d.vp; i += kStepThreads * 4) {
         int ch = -1;
         if (i < KD) ch = i < d.dp ? hk * d.dp + i : -1;
         else if (i < 2 * KD) ch = i - KD < d.dp ? d.col_k() + hk * d.dp + i - KD : -1;
         else ch = d.col_v() + h * d.vp + i - 2 * KD;
-        float y = 0.f;
+        float4 y = float4{0.f, 0.f, 0.f, 0.f};
         if (ch >= 0) {
-            y = siluf(short_conv(p.conv_w, proj, 0, ring, ch, d.conv(), d.taps, 0, past));
-            if (keeps || i >= 2 * KD) ring[(size_t)(past % d.taps) * d.conv() + ch] = proj[ch];
+            y = silu4(short_conv4(p.conv_w, proj, 0, ring, ch, d.conv(), d.taps, 0, past));
+            if (keeps || i >= 2 * KD) *(float4 *)(ring + (size_t)(past % d.taps) * d.conv() + ch) = *(const float4 *)(proj + ch);
         }
-        if (i < 2 * KD) qs[i] = y;  // (ks follows qs)
-        else vs[i - 2 * KD] = y;
+        *(float4 *)(i < 2 * KD ? qs + i : vs + i - 2 * KD) = y;  // (ks follows qs)
     }
     __syncthreads();
     if (wave < 2) {
@@ -191,10 +190,8 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(DeltaParams p)
 struct MemoryGates {
     float in, forget;
 };
-template <typename T> __device__ inline MemoryGates memory_gates(const MemoryParams &p, const float *proj, int r) {
-    const float zi = (proj[p.d.mem_i() + r] + Elem<T>::ld((const T *)p.i_bias, r)) / p.cap;
-    const float zf = (proj[p.d.mem_f() + r] + Elem<T>::ld((const T *)p.f_bias, r)) / p.cap;
-    return MemoryGates{p.cap * tanhf(zi), -softplusf(-p.cap * tanhf(zf))};
+__device__ inline MemoryGates memory_gates(float cap, float zi, float zf) {
+    return MemoryGates{cap * tanhf(zi / cap), -softplusf(-cap * tanhf(zf / cap))};
 }
 
 template <typename T, int LC, int RP>
@@ -213,7 +210,7 @@ __device__ inline void memory_step(const MemoryParams &p, int head, int b, float
     };
     request(0);
     const float m_old = past ? *mx : 0.f;
-    const MemoryGates gt = memory_gates<T>(p, proj, head);
+    const MemoryGates gt = memory_gates(p.cap, proj[d.mem_i() + head] + Elem<T>::ld((const T *)p.i_bias, head), proj[d.mem_f() + head] + Elem<T>::ld((const T *)p.f_bias, head));
     const float m_new = fmaxf(gt.forget + m_old, gt.in), keep = expf(gt.forget + m_old - m_new), put = expf(gt.in - m_new);
     for (int i = tid; i < 2 * KD; i += kStepThreads) {
         const int c = i < KD ? i : i - KD;
@@ -268,10 +265,18 @@ template <typename T> __device__ inline void memory_gate_scan(const MemoryParams
     const int lane = threadIdx.x & 63;
     float *mx = p.state + (size_t)b * p.state_stride + d.st_max() + head;
     float m = *p.d_past ? *mx : 0.f;
+    auto row_at = [&](int t0) { return (size_t)b * p.S + min(t0 + lane, p.S - 1); };
+    auto raw = [&](int t0) {
+        const float *proj = p.proj + row_at(t0) * d.n_in();
+        return float2{proj[d.mem_i() + head], proj[d.mem_f() + head]};
+    };
+    const float ib = Elem<T>::ld((const T *)p.i_bias, head), fb = Elem<T>::ld((const T *)p.f_bias, head);
+    float2 next = raw(0);
     for (int t0 = 0; t0 < p.S; t0 += 64) {
         const int n = min(64, p.S - t0);
-        const size_t row = (size_t)b * p.S + min(t0 + lane, p.S - 1);
-        const MemoryGates gt = memory_gates<T>(p, p.proj + row * d.n_in(), head);
+        const size_t row = row_at(t0);
+        const MemoryGates gt = memory_gates(p.cap, next.x + ib, next.y + fb);
+        next = raw(t0 + 64);
         float f = gt.forget, i = gt.in;
 #pragma unroll
         for (int off = 1; off < 64; off <<= 1) {
@@ -288,18 +293,18 @@ template <typename T> __device__ inline void memory_gate_scan(const MemoryParams
     if (lane == 0) *mx = m;
 }
 
-// workgroups 2 row, 2 row + 1: queries and keys of a row of the attention; then one per (sequence, memory head)
+// one workgroup per (sequence, memory head), then two per row: queries and keys of the attention
 template <typename T, bool STEP, int LC, int RP>
 __global__ __launch_bounds__(STEP ? kStepThreads : 256) void parallel_prepare_kernel(WindowAttnParams a, MemoryParams m) {
     constexpr int NT = STEP ? kStepThreads : 256;
     extern __shared__ __align__(16) float sm[];
     __shared__ float red[NT / 64];
-    const int rows = a.B * a.S, id = blockIdx.x;
-    if (id < 2 * rows) {
-        window_prepare_row<T, NT>(a, id >> 1, id & 1, sm, red);
+    const int heads = a.B * a.d.R, id = blockIdx.x;
+    if (id >= heads) {
+        window_prepare_row<T, NT>(a, (id - heads) >> 1, (id - heads) & 1, sm, red);
         return;
     }
-    const int head = (id - 2 * rows) % a.d.R, b = (id - 2 * rows) / a.d.R;
+    const int head = id % a.d.R, b = id / a.d.R;
     if constexpr (STEP) memory_step<T, LC, RP>(m, head, b, sm, red);
     else if (threadIdx.x < 64) memory_gate_scan<T>(m, head, b);
 }
@@ -368,10 +373,9 @@ template <typename T> __global__ __launch_bounds__(256) void delta_prepare_kerne
     const DeltaDims &d = p.d;
     const int row = blockIdx.x, b = row / p.S, s = row % p.S, past = *p.d_past, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const float *proj = p.proj + (size_t)row * d.n_in(), *ring = p.state + (size_t)b * p.state_stride + d.st_ring();
-    for (int ch = tid; ch < d.conv(); ch += 256) {
-        const float y = siluf(short_conv(p.conv_w, proj, d.n_in(), ring, ch, d.conv(), d.taps, s, past));
-        if (ch < d.col_v()) buf[ch] = y;
-        else p.v[(size_t)row * d.H * d.vp + ch - d.col_v()] = y;
+    for (int ch = tid * 4; ch < d.conv(); ch += 1024) {
+        const float4 y = silu4(short_conv4(p.conv_w, proj, d.n_in(), ring, ch, d.conv(), d.taps, s, past));
+        *(float4 *)(ch < d.col_v() ? buf + ch : p.v + (size_t)row * d.H * d.vp + ch - d.col_v()) = y;
     }
     for (int h = tid; h < d.H; h += 256) p.beta[(size_t)row * d.H + h] = sigmoidf(proj[d.col_b() + h]);
     for (int i = tid; i < d.low(); i += 256) Elem<T>::st((T *)p.low, (size_t)row * d.low() + i, proj[d.col_low() + i]);
@@ -591,7 +595,7 @@ struct RecurrenceParams {
 // v_mfma_f32_16x16x4_f32 (lane (quad, c): channels 4 quad .. + 3 of a tile, column c).  An accumulator register is at the
 // same time the second operand of the next product, over the four channels 4 quad + i.
 template <bool DELTA, int TW>
-__global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
+__global__ __launch_bounds__(256, 1) void recurrence_kernel(RecurrenceParams p) {
     constexpr int KD = 64 * TW;
     __shared__ __align__(16) float4 part[2][4][2][64];
     typedef float f4_t __attribute__((ext_vector_type(4)));
@@ -612,23 +616,26 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
         f4_t qt[TW], kt[DELTA ? TW : 1], kh[TW], gam[TW], B, T;
         float v[4];
     };
+    // (a uniform base and a 32-bit offset of the lane per load, no branches: the waits then count loads exactly)
+    const unsigned at_row = (unsigned)(c16 * KD + k0 + 4 * quad), at_key = (unsigned)((k0 + c16) * kBlock + 4 * quad), at_tok = (unsigned)(c16 * kBlock + 4 * quad);
+    const bool has_value = col < p.nv;
+    const float *values = p.v + row0 * p.ldv + h * p.vp;
+    const unsigned vcol = (unsigned)min(col, p.nv - 1);
     auto request = [&](Block &x, int n) {
-        const size_t blk = blk0 + min(n, nb - 1);
+        const int nn = min(n, nb - 1);
+        const size_t blk = blk0 + nn;
+        const float *qt = op.qt + blk * kBlock * KD, *kt = op.kt + blk * kBlock * KD, *kh = op.kh + blk * kBlock * KD, *gam = op.gam + blk * KD;
 #pragma unroll
         for (int t = 0; t < TW; t++) {
-            const int c = k0 + 16 * t;
-            x.qt[t] = *(const f4_t *)(op.qt + (blk * kBlock + c16) * KD + c + 4 * quad);
-            if constexpr (DELTA) x.kt[t] = *(const f4_t *)(op.kt + (blk * kBlock + c16) * KD + c + 4 * quad);
-            x.kh[t] = *(const f4_t *)(op.kh + (blk * KD + c + c16) * kBlock + 4 * quad);
-            x.gam[t] = *(const f4_t *)(op.gam + blk * KD + c + 4 * quad);
+            x.qt[t] = *(const f4_t *)(qt + at_row + 16 * t);
+            if constexpr (DELTA) x.kt[t] = *(const f4_t *)(kt + at_row + 16 * t);
+            x.kh[t] = *(const f4_t *)(kh + at_key + 16 * t * kBlock);
+            x.gam[t] = *(const f4_t *)(gam + k0 + 16 * t + 4 * quad);
         }
-        x.B = *(const f4_t *)(op.B + (blk * kBlock + c16) * kBlock + 4 * quad);
-        if constexpr (DELTA) x.T = *(const f4_t *)(op.T + (blk * kBlock + c16) * kBlock + 4 * quad);
+        x.B = *(const f4_t *)(op.B + blk * kBlock * kBlock + at_tok);
+        if constexpr (DELTA) x.T = *(const f4_t *)(op.T + blk * kBlock * kBlock + at_tok);
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int t = min(min(n, nb - 1) * kBlock + 4 * quad + i, p.S - 1);
-            x.v[i] = col < p.nv ? p.v[(row0 + t) * p.ldv + h * p.vp + col] : 1.f;
-        }
+        for (int i = 0; i < 4; i++) x.v[i] = values[(size_t)min(nn * kBlock + 4 * quad + i, p.S - 1) * p.ldv + vcol];
     };
     auto step = [&](const Block &x, int n) {
         f4_t pq = {0.f, 0.f, 0.f, 0.f}, pk = pq;
@@ -645,23 +652,27 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
 #pragma unroll
         for (int t = 0; t < TW; t++) S[t] *= x.gam[t];
         __syncthreads();  // (the other half of `part` was read before the barrier of the block before)
-        f4_t u;
-        if constexpr (DELTA) {
-            f4_t r = {x.v[0], x.v[1], x.v[2], x.v[3]};
+        f4_t u, val;
 #pragma unroll
-            for (int w = 0; w < 4; w++) r -= __builtin_bit_cast(f4_t, part[n & 1][w][1][lane]);
+        for (int i = 0; i < 4; i++) val[i] = has_value ? x.v[i] : 1.f;
+        if constexpr (DELTA) {
+            f4_t sum[4];
+#pragma unroll
+            for (int w = 0; w < 4; w++) sum[w] = __builtin_bit_cast(f4_t, part[n & 1][w][1][lane]);
+            const f4_t r = val - ((sum[0] + sum[1]) + (sum[2] + sum[3]));
             u = f4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int i = 0; i < 4; i++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(x.T[i], r[i], u, 0, 0, 0);
-        } else u = f4_t{x.v[0], x.v[1], x.v[2], x.v[3]};
+        } else u = val;
 #pragma unroll
         for (int t = 0; t < TW; t++)
 #pragma unroll
             for (int i = 0; i < 4; i++) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kh[t][i], u[i], S[t], 0, 0, 0);
         if (wave == (n & 3)) {
-            f4_t out = {0.f, 0.f, 0.f, 0.f};
+            f4_t sum[4];
 #pragma unroll
-            for (int w = 0; w < 4; w++) out += __builtin_bit_cast(f4_t, part[n & 1][w][0][lane]);
+            for (int w = 0; w < 4; w++) sum[w] = __builtin_bit_cast(f4_t, part[n & 1][w][0][lane]);
+            f4_t out = (sum[0] + sum[1]) + (sum[2] + sum[3]);
 #pragma unroll
             for (int i = 0; i < 4; i++) out = __builtin_amdgcn_mfma_f32_16x16x4f32(x.B[i], u[i], out, 0, 0, 0);
             if (col < p.ncol)
@@ -672,14 +683,18 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
                 }
         }
     };
-    Block x, y;
-    request(x, 0);
-    for (int n = 0; n < nb; n += 2) {
-        request(y, n + 1);
-        step(x, n);
-        if (n + 1 >= nb) break;
-        request(x, n + 2);
-        step(y, n + 1);
+    // the operands of the next AHEAD - 1 blocks are on their way while one is worked on
+    constexpr int AHEAD = TW <= 2 ? 4 : TW <= 4 ? 3 : 2;
+    Block x[AHEAD];
+#pragma unroll
+    for (int i = 0; i + 1 < AHEAD; i++) request(x[i], i);
+    for (int n0 = 0; n0 < nb; n0 += AHEAD) {
+#pragma unroll
+        for (int i = 0; i < AHEAD; i++) {
+            if (n0 + i >= nb) break;
+            request(x[(i + AHEAD - 1) % AHEAD], n0 + i + AHEAD - 1);
+            step(x[i], n0 + i);
+        }
     }
     if (col < p.ncol)
 #pragma unroll
@@ -763,7 +778,7 @@ struct HeadOutParams {
     const int32_t *d_past;
 };
 template <typename T> __global__ __launch_bounds__(256) void head_out_kernel(HeadOutParams p) {
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int tid = threadIdx.x;
     if ((int)blockIdx.x >= p.rows) {
         // the portion's last taps - 1 projected values of sequence b, column by column
         const int tail = min(p.taps - 1, p.S), per = (p.channels + 255) / 256, id = blockIdx.x - p.rows, b = id / per, ch = id % per * 256 + tid;
@@ -774,20 +789,41 @@ template <typename T> __global__ __launch_bounds__(256) void head_out_kernel(Hea
         }
         return;
     }
-    const int row = blockIdx.x;
-    for (int h = wave; h < p.H; h += 4) {
-        const float *o = p.o + ((size_t)row * p.H + h) * p.op;
-        float den = 1.f, ss = 0.f;
-        if (p.den) den = 1.0f / (fmaxf(fabsf(o[p.v]), p.den[((size_t)row * p.H + h) * 4 + 2]) + 1e-6f);
-        for (int c = lane; c < p.v; c += 64) {
-            const float x = o[c] * den;
-            ss = fmaf(x, x, ss);
-        }
-        const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)p.v + p.eps) * den;
+    // 32 lanes per head; a head of up to 128 values stays in registers
+    const int row = blockIdx.x, sub = tid & 31;
+    for (int h0 = 0; h0 < p.H; h0 += 8) {
+        const int h = min(h0 + (tid >> 5), p.H - 1);  // (the last head again: the same values)
+        const float *o = p.o + ((size_t)row * p.H + h) * p.op, *g = p.gate + row * p.ld_gate + h * p.vp;
         const T *nw = (const T *)p.norm + h * p.norm_stride;
-        const float *g = p.gate + row * p.ld_gate + h * p.vp;
         T *out = (T *)p.out + row * p.ld_out + h * p.vp;
-        for (int c = lane; c < p.vp; c += 64) Elem<T>::st(out, c, c < p.v ? o[c] * inv * Elem<T>::ld(nw, c) * sigmoidf(g[c]) * p.scale : 0.f);
+        float den = 1.f, ss = 0.f;
+        auto row4 = [&](int c) {  // (columns past v: zeros)
+            float4 x = *(const float4 *)(o + c);
+            float *f = (float *)&x;
+#pragma unroll
+            for (int e = 0; e < 4; e++) f[e] = c + e < p.v ? f[e] : 0.f;
+            return x;
+        };
+        const int c0 = sub * 4, first = min(c0, p.vp - 4);
+        const float4 x0 = row4(first), z0 = *(const float4 *)(g + first);
+        Load4<T> w0;
+        w0.get(nw + first);
+        if (p.den) den = 1.0f / (fmaxf(fabsf(o[p.v]), p.den[((size_t)row * p.H + h) * 4 + 2]) + 1e-6f);
+        for (int c = c0; c < p.vp; c += 128) {
+            const float4 x = c == c0 ? x0 : row4(c);
+            ss = fmaf(x.x, x.x, fmaf(x.y, x.y, fmaf(x.z, x.z, fmaf(x.w, x.w, ss))));
+        }
+        const float inv = 1.0f / sqrtf(group_sum<32>(ss) * den * den / (float)p.v + p.eps) * den * p.scale;
+        for (int c = c0; c < p.vp; c += 128) {
+            float4 x = c == c0 ? x0 : row4(c);
+            const float4 z = c == c0 ? z0 : *(const float4 *)(g + c);
+            Load4<T> wl = w0;
+            if (c != c0) wl.get(nw + c);
+            float w[4];
+            wl.widen(w);
+            x.x *= inv * w[0] * sigmoidf(z.x); x.y *= inv * w[1] * sigmoidf(z.y); x.z *= inv * w[2] * sigmoidf(z.z); x.w *= inv * w[3] * sigmoidf(z.w);
+            store4<T>(out + c, x);
+        }
     }
 }
 static int head_out(const HeadOutParams &p, int B, int dtype, hipStream_t s) {

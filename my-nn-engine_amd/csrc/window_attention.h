@@ -1,6 +1,7 @@
 // Attention over the last `window` tokens and a sequence's first keep_first (window_attention.hip): grouped queries, values
 // that are the keys before norm and rotation, a short convolution over time in front of both.
 #pragma once
+#include "dense_load.h"
 #include "dense.h"
 #include "model_spec.h"
 
@@ -28,16 +29,17 @@ struct WindowAttnParams {
 };
 
 #ifdef __HIPCC__
-// Channel ch of the short convolution at token s of a portion that starts at position `past`: tokens before the portion are
-// in the ring.  Zeros before the sequence.
-__device__ inline float short_conv(const float *w, const float *proj, long ld, const float *ring, int ch, int channels, int taps, int s, int past) {
-    float y = 0.f;
+// Channels ch .. ch + 3 of the short convolution at token s of a portion that starts at position `past`: tokens before the
+// portion are in the ring.  Zeros before the sequence.
+__device__ inline float4 short_conv4(const float *w, const float *proj, long ld, const float *ring, int ch, int channels, int taps, int s, int past) {
+    float4 y = float4{0.f, 0.f, 0.f, 0.f};
     for (int j = 0; j < taps; j++) {
         const int back = taps - 1 - j, at = past + s - back;
-        float u = 0.f;
-        if (s >= back) u = proj[-(long)back * ld + ch];
-        else if (at >= 0) u = ring[(size_t)(at % taps) * channels + ch];
-        y = fmaf(w[(size_t)j * channels + ch], u, y);
+        float4 u = float4{0.f, 0.f, 0.f, 0.f};
+        if (s >= back) u = *(const float4 *)(proj - (long)back * ld + ch);
+        else if (at >= 0) u = *(const float4 *)(ring + (size_t)(at % taps) * channels + ch);
+        const float4 c = *(const float4 *)(w + (size_t)j * channels + ch);
+        y.x = fmaf(c.x, u.x, y.x); y.y = fmaf(c.y, u.y, y.y); y.z = fmaf(c.z, u.z, y.z); y.w = fmaf(c.w, u.w, y.w);
     }
     return y;
 }
@@ -55,12 +57,12 @@ __device__ inline void window_prepare_row(const WindowAttnParams &p, int row, in
     float *ring = p.ring + (size_t)b * p.state_stride;
     T *dst = which ? (T *)p.cache + window_cache_row(p, b, pos) * d.row() : (T *)p.q + (size_t)row * d.qcols();
     float ss = 0.f;
-    for (int c = tid; c < nch; c += NT) {
-        const float y = short_conv(p.conv_w, proj, d.n_in(), ring, col0 + c, channels, d.taps, s, past);
-        if (p.S == 1) ring[(size_t)(pos % d.taps) * channels + col0 + c] = proj[col0 + c];
-        if (which) Elem<T>::st(dst, d.G * d.dimp + c, y);
-        buf[c] = y;
-        ss = fmaf(y, y, ss);
+    for (int c = tid * 4; c < nch; c += NT * 4) {
+        const float4 y = short_conv4(p.conv_w, proj, d.n_in(), ring, col0 + c, channels, d.taps, s, past);
+        if (p.S == 1) *(float4 *)(ring + (size_t)(pos % d.taps) * channels + col0 + c) = *(const float4 *)(proj + col0 + c);
+        if (which) store4<T>(dst + d.G * d.dimp + c, y);
+        *(float4 *)(buf + c) = y;
+        ss = fmaf(y.x, y.x, fmaf(y.y, y.y, fmaf(y.z, y.z, fmaf(y.w, y.w, ss))));
     }
     ss = wave_sum(ss);
     if ((tid & 63) == 0) red[tid >> 6] = ss;
@@ -70,18 +72,25 @@ __device__ inline void window_prepare_row(const WindowAttnParams &p, int row, in
     for (int w = 0; w < NT / 64; w++) t += red[w];
     const float inv = 1.0f / sqrtf(t / (float)(heads * d.dim) + p.eps);
     const T *nw = (const T *)(which ? p.k_norm : p.q_norm);
-    const int half = p.rot_dims / 2, pairs = d.dimp / 2;
-    for (int j = tid; j < nch / 2; j += NT) {
-        const int i = j % pairs;
-        float u = buf[2 * j] * inv * Elem<T>::ld(nw, 2 * j), v = buf[2 * j + 1] * inv * Elem<T>::ld(nw, 2 * j + 1);
+    const int half = p.rot_dims / 2;
+    for (int c = tid * 4; c < nch; c += NT * 4) {
+        const int i = c % d.dimp / 2;
+        float4 x = *(const float4 *)(buf + c);
+        Load4<T> wl;
+        wl.get(nw + c);
+        float f[4];
+        wl.widen(f);
+        x.x *= inv * f[0]; x.y *= inv * f[1]; x.z *= inv * f[2]; x.w *= inv * f[3];
+        const float2 *cs = p.rot + (size_t)pos * half;
         if (i < half) {
-            const float2 cs = p.rot[(size_t)pos * half + i];
-            const float a = u * cs.x - v * cs.y;
-            v = v * cs.x + u * cs.y;
-            u = a;
+            const float2 t2 = cs[i];
+            x = float4{x.x * t2.x - x.y * t2.y, x.y * t2.x + x.x * t2.y, x.z, x.w};
         }
-        Elem<T>::st(dst, 2 * j, u);
-        Elem<T>::st(dst, 2 * j + 1, v);
+        if (i + 1 < half) {
+            const float2 t2 = cs[i + 1];
+            x = float4{x.x, x.y, x.z * t2.x - x.w * t2.y, x.w * t2.x + x.z * t2.y};
+        }
+        store4<T>(dst + c, x);
     }
 }
 #endif
